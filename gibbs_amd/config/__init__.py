@@ -5,6 +5,7 @@ from .zokepel import ZokepelConfig
 from .rukosun import RukosunConfig
 from .ruzinex import RuzinexConfig
 from .litizen import LitizenConfig
+from .gumozen import GumozenConfig
 from .registry import (Architecture, architectures, config_from_dict,
                        find_architecture, register_architecture)
 from .spec import (ConnectionSpec, EmbeddingTablesSpec, FeedForwardSpec, LayerSpec, MixerSpec, ModelSpec, NormSpec,
@@ -15,3 +16,4 @@ register_architecture("Zokepel", ZokepelConfig, aliases=("zokepel",))
 register_architecture("Rukosun", RukosunConfig, aliases=("rukosun",))
 register_architecture("Ruzinex", RuzinexConfig, aliases=("ruzinex",))
 register_architecture("Litizen", LitizenConfig, aliases=("litizen",))
+register_architecture("Gumozen", GumozenConfig, aliases=("gumozen",))

@@ -16,12 +16,14 @@ from typing import Any, Mapping, Optional, Sequence, Tuple, Union
 @dataclass(frozen=True)
 class NormSpec:
     """A normalisation over the last axis. `kind` selects the part (`"rms"`; `"layer"`: mean taken off, gain and bias;
-    `"group_rms"`: the row in `groups` equal consecutive parts, each divided by its own root mean square)."""
+    `"group_rms"`: the row in `groups` equal consecutive parts, each divided by its own root mean square).  `scale` names a
+    further vector per channel that multiplies the normed row (a layer scale)."""
     kind: str
     eps: float
     weight: str                     # tensor name of the gain
     bias: Optional[str] = None      # tensor name of the bias (kinds that have one)
     groups: int = 1                 # parts of the row that are normed by themselves (kind "group_rms")
+    scale: Optional[str] = None     # tensor name of a further scale per channel (kind "rms")
 
 
 @dataclass(frozen=True)
@@ -146,6 +148,7 @@ class ModelSpec:
     # (`embedding_position`, kind "sinusoidal" with its `base`; None: none).  `reinject_before`: runs of the
     # order (indices into `order`) right before which the embedding's output is added into the stream again.
     embedding_scale: float = 1.0
+    embedding_norm: Optional[NormSpec] = None      # the table's row is normed (kind "rms"); the stream starts as the result
     embedding_position: Optional[PositionSpec] = None
     reinject_before: Tuple[int, ...] = ()
     # Tables whose rows are added to the token table's (hashed token pairs, learned positions), and the number of

@@ -90,6 +90,30 @@ int gibbs_qkv_prepare_full(void* rows, long ld, void* kpages, void* vpages, int 
                            float qk_eps, int norm_dim, int v_from_k, const float* v_inv_freq, int v_rot, hipStream_t stream);
 int gibbs_attention_finish(void* att, long ldo, const void* gate, long ld_gate, int gate_head, int dtype, const int* pos,
                            const float* v_inv_freq, int v_rot, int variant, int n_rows, int nh, int vd, int vt, hipStream_t stream);
+// ---- stream_rows.hip: readers of the residual stream without a norm, the normed embedding
+int gibbs_embed_norm(const void* table, int dtype, const int* ids, float* x, const float* gain, float eps, int n, int hidden, int vocab,
+                     hipStream_t stream);
+int gibbs_stream_rows(const float* x, void* out, int dtype, long count, hipStream_t stream);
+int gibbs_stream_shift(const float* x, const float* mu, float* state, long slot_stride, const int* row_req, const int* cu, const int* slot,
+                       void* out, int dtype, int n_rows, int hidden, hipStream_t stream);
+int gibbs_rmsnorm_rows_add_read(float* x, const void* in, int parts, long part_stride, const int* place, const float* weight, int top,
+                                const void* shared, const float* gate, const float* gain, float eps, int read, const float* mu, float* state,
+                                long slot_stride, const int* slot, void* out, int dtype, int n, int hidden, hipStream_t stream);
+// ---- diff_attention.hip: rows and heads of a differential attention
+int gibbs_diff_prepare(const void* rows, long ld, void* q_out, void* kpages, void* vpages, int dtype, const float* q_gain,
+                       const float* k_gain, float eps, const float* inv_freq, int rot, int variant, const float* cs_table, int table_len,
+                       const int* pos, const int* row_req, const int* table, int max_pages, int page_size, int num_pages, int n_rows,
+                       int H, int G, int dim, int vdim, int ks, int vs, hipStream_t stream);
+int gibbs_diff_finish(const void* att, int vs, const void* gate, long ld_gate, const float* lambda, float eps, float out_scale, void* o,
+                      int dtype, int n_rows, int H, int V, hipStream_t stream);
+// ---- gated_outer.hip: the gated outer-product recurrence
+int gibbs_gated_outer_prep(const void* raw, long ld, int dtype, const float* bias, const float* lower, float* q, float* f, float* k,
+                           float* v, int n_rows, int H, int D, int V, hipStream_t stream);
+int gibbs_gated_outer_step_takes(int D, int V);
+int gibbs_gated_outer_step(const void* raw, long ld, int dtype, const float* bias, const float* lower, const float* gain, float eps,
+                           float* state, long slot_stride, const int* slot, void* out, int n_req, int H, int D, int V, hipStream_t stream);
+int gibbs_gated_outer_rule(const float* q, const float* k, const float* v, const float* decay, float* state, long slot_stride,
+                           const int* cu, const int* slot, float* out, int n_req, int H, int D, int V, hipStream_t stream);
 // ---- moe.hip: mixture of experts
 long gibbs_moe_capacity(int n_pairs, int E, int bm);
 int gibbs_moe_tile(int n_pairs, int E);
@@ -103,6 +127,9 @@ int gibbs_moe_group(const int* chosen, int n_pairs, int E, int bm, int* sorted_p
                     hipStream_t stream);
 int gibbs_moe_gemm(const void* X, long ldx, int top, const int* sorted_pair, const int* tile_expert, long cap, int bm,
                    const void* w_a, const void* w_b, void* Y, long ldy, int dtype, int O, int I, int act, hipStream_t stream);
+int gibbs_moe_gemm_weighted(const void* X, long ldx, int top, const int* sorted_pair, const int* tile_expert, long cap, int bm,
+                            const void* w_a, const void* w_b, const float* in_weight, void* Y, long ldy, int dtype, int O, int I, int act,
+                            hipStream_t stream);
 int gibbs_moe_combine(const void* y, const int* pair_pos, const float* weight, const void* shared, const float* sgate, void* out,
                       int dtype, int n, int top, int W, hipStream_t stream);
 int gibbs_causal_conv_silu(const void* in, long ld, int dtype, const float* taps, float* state, long slot_stride,

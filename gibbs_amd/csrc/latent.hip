@@ -254,7 +254,7 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(const T* __restrict
                                                              int page_size, int num_pages, int nh, int dim, int rot, int rank) {
   const int n = blockIdx.x, lane = threadIdx.x % WAVE;
   const int p = pos[n];
-  if (threadIdx.x < WAVE) {
+  if (threadIdx.x < WAVE && kv) {      // (kv null: another layer's cached rows are read, only the queries are prepared)
     int page = table[(size_t)row_req[n] * max_pages + p / page_size];
     page = page < 0 ? 0 : (page >= num_pages ? num_pages - 1 : page);      // never write outside the pool
     T* dst = pages + ((size_t)page * page_size + p % page_size) * (rank + rot);
@@ -635,7 +635,7 @@ GIBBS_EXPORT int gibbs_latent_prepare(const void* kv, long ld_kv, const void* q,
   GIBBS_REQUIRE(n_rows >= 0 && nh > 0 && dim >= 0 && rot >= 0 && rank > 0, "latent_prepare: bad sizes rows=%d heads=%d dim=%d rot=%d rank=%d", n_rows, nh, dim, rot, rank);
   GIBBS_REQUIRE(rot_dims >= 0 && rot_dims <= rot && rot_dims % 2 == 0 && (rot_dims == 0 || inv_freq), "latent_prepare: %d rotated dimensions of %d", rot_dims, rot);
   GIBBS_REQUIRE(variant == 0 || variant == 1, "latent_prepare: unknown pairing %d", variant);
-  GIBBS_REQUIRE(ld_kv >= rank + rot && ld_q >= (long)nh * (dim + rot) && ld_qo >= (long)nh * (rank + rot), "latent_prepare: row strides shorter than rows");
+  GIBBS_REQUIRE((!kv || ld_kv >= rank + rot) && ld_q >= (long)nh * (dim + rot) && ld_qo >= (long)nh * (rank + rot), "latent_prepare: row strides shorter than rows");
   GIBBS_REQUIRE(page_size > 0 && max_pages > 0 && num_pages > 0, "latent_prepare: bad cache geometry");
   if (n_rows == 0) return 0;
   const dim3 grid(n_rows);

@@ -4,13 +4,15 @@
 //   route      z = W_r h + b in float32 (h as the step holds it); the `top` largest logits (the lower index among
 //              equals); weights = softmax over the chosen logits alone; gate = sigmoid(w_sg . h) for the shared expert
 //              (mode 1: scores s = softmax(z) over all router outputs; the `top` largest of s + correction; weights = the
-//              chosen scores s divided by their sum + 1e-20.  Router outputs from `E_real` on are identity experts: they
+//              chosen scores s divided by their sum + 1e-20; mode 2: scores s = sigmoid(z), the `top` largest of s +
+//              correction, or of z without one, weights = the chosen scores s as they are.  Router outputs from `E_real` on are identity experts: they
 //              have no matrices, their result is the row itself, and their pairs take no place in the tiles)
 //   group      the step's (row, choice) pairs sorted by expert into tiles of `bm` pairs that belong to one expert
 //              each (every expert's stretch is padded to whole tiles); nothing goes back to the host, so a step
 //              with experts can be captured in a graph: the products below run over the worst-case number of tiles
 //              and a tile without an expert returns at once
-//   gate_up    act[m] = activation(W_gate,e h[row(m)]) * (W_up,e h[row(m)]) for every sorted pair m (rows gathered)
+//   gate_up    act[m] = activation(W_gate,e h[row(m)]) * (W_up,e h[row(m)]) for every sorted pair m (rows gathered);
+//              with the pairs' weights on their inputs, both products' float32 sums times the pair's weight first
 //   down       y[m] = W_down,e act[m]
 //   combine    out[row] = sum_c weight[row][c] y[place(row, c)] (ascending c) + gate[row] shared[row], float32 sums
 //
@@ -110,7 +112,7 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(const T* __restrict__ h
                                                         const float* __restrict__ router_bias, const float* __restrict__ shared_gate,
                                                         int* __restrict__ chosen, float* __restrict__ weight, float* __restrict__ sgate,
                                                         int W, int E, int top, int mode) {
-  extern __shared__ float z[];   // [E] (mode 1: and the scores behind them, [E])
+  extern __shared__ float z[];   // [E] (mode 1 and 2: and the scores behind them, [E])
   const int n = blockIdx.x, wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE, n_waves = blockDim.x / WAVE;
   const T* row = h + (size_t)n * ldh;
   const bool vec = W % 4 == 0 && ldh % 4 == 0 && ((uintptr_t)h % 16) == 0 && ((uintptr_t)router % 16) == 0 && ((uintptr_t)shared_gate % 16) == 0;
@@ -142,6 +144,14 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(const T* __restrict__ h
   int* mine = chosen + (size_t)n * top;
   float* wts = weight + (size_t)n * top;
   float* score = z + E;
+  if (mode == 2 && router_bias) {
+    for (int e = lane; e < E; e += WAVE) {
+      score[e] = 1.0f / (1.0f + expf(-z[e]));
+      z[e] = score[e] + router_bias[e];
+    }
+    __builtin_amdgcn_s_waitcnt(0);
+    __builtin_amdgcn_wave_barrier();
+  }
   if (mode == 1) {
     // scores over all outputs; what is compared is the score plus the output's correction
     float zmax = -INFINITY;
@@ -181,7 +191,8 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(const T* __restrict__ h
       pv = -INFINITY;
     }
     if (c == 0) best = pv;
-    const float w = mode == 1 ? score[pick] : (pv == -INFINITY ? 0.f : expf(pv - best));
+    const float w = (mode == 1 || (mode == 2 && router_bias)) ? score[pick]
+                    : (pv == -INFINITY ? 0.f : (mode == 2 ? 1.0f / (1.0f + expf(-pv)) : expf(pv - best)));
     sum += w;
     if (lane == 0) {
       mine[c] = pick;
@@ -191,7 +202,7 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(const T* __restrict__ h
     __builtin_amdgcn_s_waitcnt(0);   // (the wave's own LDS write above is read by its next scan)
     __builtin_amdgcn_wave_barrier();
   }
-  if (lane == 0) {
+  if (lane == 0 && mode != 2) {
     if (mode == 1)
       for (int c = 0; c < top; ++c) wts[c] = wts[c] / (sum + 1e-20f);
     else
@@ -256,7 +267,7 @@ template <typename T, int BM, bool GLU>
 __global__ __launch_bounds__(256) void moe_gemm_plain_kernel(const T* __restrict__ X, long ldx, int top, const int* __restrict__ sorted_pair,
                                                              const int* __restrict__ tile_expert, const T* __restrict__ Wa,
                                                              const T* __restrict__ Wb, long expert_stride, T* __restrict__ Y, long ldy,
-                                                             int O, int I, int act) {
+                                                             int O, int I, int act, const float* __restrict__ in_weight) {
   constexpr int TK = 16, RPT = BM / 4;
   __shared__ float sx[TK][BM + 1];
   __shared__ float sa[TK][64 + 1];
@@ -302,7 +313,8 @@ __global__ __launch_bounds__(256) void moe_gemm_plain_kernel(const T* __restrict
   for (int r = 0; r < RPT; ++r) {
     const int row = ty + 4 * r;
     if (src[row] < 0) continue;
-    const float v = GLU ? activate(acc_a[r], act) * acc_b[r] : acc_a[r];
+    const float w = (GLU && in_weight) ? in_weight[sorted_pair[tile * BM + row]] : 1.f;
+    const float v = GLU ? activate(w * acc_a[r], act) * (w * acc_b[r]) : acc_a[r];
     Y[(size_t)(tile * BM + row) * ldy + col0 + tx] = from_float<T>(v);
   }
 }
@@ -322,7 +334,7 @@ template <bool GLU>
 __global__ __launch_bounds__(256) void moe_gemm_few_kernel(const bf16* __restrict__ X, long ldx, int top, const int* __restrict__ sorted_pair,
                                                            const int* __restrict__ tile_expert, const bf16* __restrict__ Wa,
                                                            const bf16* __restrict__ Wb, long expert_stride, bf16* __restrict__ Y, long ldy,
-                                                           int O, int I, int act) {
+                                                           int O, int I, int act, const float* __restrict__ in_weight) {
   constexpr int NF = 2, NA = GLU ? 2 * NF : NF;    // feature tiles of 16 a workgroup; accumulators a wave
   __shared__ float part[4][NA][WAVE][4];
   const int tile = blockIdx.y, e = tile_expert[tile];
@@ -371,6 +383,7 @@ __global__ __launch_bounds__(256) void moe_gemm_few_kernel(const bf16* __restric
     for (int i = 0; i < 4; ++i) part[wave][t][lane][i] = acc[t][i];
   __syncthreads();
   if (wave != 0 || src < 0) return;
+  const float pw = (GLU && in_weight) ? in_weight[pair] : 1.f;
 #pragma unroll
   for (int t = 0; t < NF; ++t)
 #pragma unroll
@@ -383,7 +396,7 @@ __global__ __launch_bounds__(256) void moe_gemm_few_kernel(const bf16* __restric
         a += part[w][t][lane][i];
         if (GLU) b += part[w][NF + t][lane][i];
       }
-      Y[(size_t)place * ldy + col] = (bf16)(GLU ? activate(a, act) * b : a);
+      Y[(size_t)place * ldy + col] = (bf16)(GLU ? activate(pw * a, act) * (pw * b) : a);
     }
 }
 
@@ -401,7 +414,7 @@ template <bool GLU, int BK, int BN, int NW>
 __global__ __launch_bounds__(NW * WAVE) void moe_gemm_tiled_kernel(const bf16* __restrict__ X, long ldx, int top, const int* __restrict__ sorted_pair,
                                                              const int* __restrict__ tile_expert, const bf16* __restrict__ Wa,
                                                              const bf16* __restrict__ Wb, long expert_stride, bf16* __restrict__ Y, long ldy,
-                                                             int O, int I, int act) {
+                                                             int O, int I, int act, const float* __restrict__ in_weight) {
   using Tile = MoeTile<BK, BN>;
   constexpr int KC = BK / 8;                        // chunks of 16 bytes in a row of a tile
   constexpr int THREADS = NW * WAVE, WN = NW / 2;   // waves: 2 along the places, WN along the rows of W
@@ -411,6 +424,7 @@ __global__ __launch_bounds__(NW * WAVE) void moe_gemm_tiled_kernel(const bf16* _
   extern __shared__ __attribute__((aligned(16))) char moe_lds[];
   Tile* tiles = (Tile*)moe_lds;                     // [2]
   int* srcs = (int*)(moe_lds + 2 * sizeof(Tile));   // [TBM]
+  float* pair_w = (float*)(srcs + TBM);             // [TBM]: the pairs' weights on their inputs (1 without)
   const int tile = blockIdx.y, e = tile_expert[tile];
   if (e < 0) return;
   const int tid = threadIdx.x, wave = tid / WAVE, lane = tid % WAVE;
@@ -419,6 +433,7 @@ __global__ __launch_bounds__(NW * WAVE) void moe_gemm_tiled_kernel(const bf16* _
   if (tid < TBM) {
     const int pair = sorted_pair[tile * TBM + tid];
     srcs[tid] = pair < 0 ? -1 : (top > 0 ? pair / top : tile * TBM + tid);
+    if (GLU) pair_w[tid] = (in_weight && pair >= 0) ? in_weight[pair] : 1.f;
   }
   __syncthreads();
   const bf16* wa = Wa + (size_t)e * expert_stride;
@@ -509,10 +524,11 @@ __global__ __launch_bounds__(NW * WAVE) void moe_gemm_tiled_kernel(const bf16* _
       if (srcs[row] < 0) continue;
       bf16* y = Y + (size_t)(tile * TBM + row) * ldy;
       if (GLU) {
+        const float w = pair_w[row];
 #pragma unroll
         for (int n = 0; n < NT / 2; ++n) {
           const int col = col0 + wc[n] + lane % 32;
-          if (col < O) y[col] = (bf16)(activate(acc[m][n][i], act) * acc[m][NT / 2 + n][i]);
+          if (col < O) y[col] = (bf16)(activate(w * acc[m][n][i], act) * (w * acc[m][NT / 2 + n][i]));
         }
       } else {
 #pragma unroll
@@ -526,8 +542,8 @@ __global__ __launch_bounds__(NW * WAVE) void moe_gemm_tiled_kernel(const bf16* _
 
 template <bool GLU, int BK, int BN, int NW>
 int launch_tiled_as(const bf16* X, long ldx, int top, const int* sorted_pair, const int* tile_expert, int tiles, const bf16* wa, const bf16* wb,
-                    long stride, bf16* Y, long ldy, int O, int I, int act, hipStream_t stream) {
-  constexpr int LDS = 2 * (int)sizeof(MoeTile<BK, BN>) + TBM * (int)sizeof(int);
+                    long stride, bf16* Y, long ldy, int O, int I, int act, const float* in_weight, hipStream_t stream) {
+  constexpr int LDS = 2 * (int)sizeof(MoeTile<BK, BN>) + 2 * TBM * (int)sizeof(int);
   static bool prepared = false;    // (one flag per instantiation)
   if (!prepared) {
     hipError_t e = hipFuncSetAttribute((const void*)moe_gemm_tiled_kernel<GLU, BK, BN, NW>, hipFuncAttributeMaxDynamicSharedMemorySize, LDS);
@@ -535,17 +551,17 @@ int launch_tiled_as(const bf16* X, long ldx, int top, const int* sorted_pair, co
     prepared = true;
   }
   moe_gemm_tiled_kernel<GLU, BK, BN, NW><<<dim3(ceil_div(O, GLU ? BN / 2 : BN), tiles), NW * WAVE, LDS, stream>>>(X, ldx, top, sorted_pair, tile_expert, wa, wb,
-                                                                                                        stride, Y, ldy, O, I, act);
+                                                                                                        stride, Y, ldy, O, I, act, in_weight);
   return 0;
 }
 template <bool GLU>
 int launch_tiled(const bf16* X, long ldx, int top, const int* sorted_pair, const int* tile_expert, int tiles, const bf16* wa, const bf16* wb,
-                 long stride, bf16* Y, long ldy, int O, int I, int act, hipStream_t stream) {
+                 long stride, bf16* Y, long ldy, int O, int I, int act, const float* in_weight, hipStream_t stream) {
   // wide results with a long inner size: 256 rows of W a workgroup and 8 waves (the tile of X is read by half as many
   // workgroups); otherwise 128 rows and 4 waves, which leaves more workgroups to spread
   if (I > 1024 && O >= 512)
-    return launch_tiled_as<GLU, 32, 256, 8>(X, ldx, top, sorted_pair, tile_expert, tiles, wa, wb, stride, Y, ldy, O, I, act, stream);
-  return launch_tiled_as<GLU, 32, 128, 4>(X, ldx, top, sorted_pair, tile_expert, tiles, wa, wb, stride, Y, ldy, O, I, act, stream);
+    return launch_tiled_as<GLU, 32, 256, 8>(X, ldx, top, sorted_pair, tile_expert, tiles, wa, wb, stride, Y, ldy, O, I, act, in_weight, stream);
+  return launch_tiled_as<GLU, 32, 128, 4>(X, ldx, top, sorted_pair, tile_expert, tiles, wa, wb, stride, Y, ldy, O, I, act, in_weight, stream);
 }
 
 // ------------------------------------------------------------------------------------------------- combine
@@ -566,7 +582,7 @@ __global__ void moe_combine_kernel(const T* __restrict__ y, const int* __restric
 #pragma unroll
   for (int s = 0; s < MOST; ++s) {
     at[s] = s < top ? row_of(s) : y;
-    w[s] = s < top ? weight[(size_t)n * top + s] : 0.f;
+    w[s] = s < top ? (weight ? weight[(size_t)n * top + s] : 1.f) : 0.f;
   }
   if (VEC) {
     for (int c = threadIdx.x * 4; c < W; c += blockDim.x * 4) {
@@ -578,7 +594,7 @@ __global__ void moe_combine_kernel(const T* __restrict__ y, const int* __restric
           v.x = fmaf(w[s], r.x, v.x); v.y = fmaf(w[s], r.y, v.y); v.z = fmaf(w[s], r.z, v.z); v.w = fmaf(w[s], r.w, v.w);
         }
       for (int s = MOST; s < top; ++s) {
-        const float ws = weight[(size_t)n * top + s];
+        const float ws = weight ? weight[(size_t)n * top + s] : 1.f;
         const float4 r = load4f(row_of(s) + c);
         v.x = fmaf(ws, r.x, v.x); v.y = fmaf(ws, r.y, v.y); v.z = fmaf(ws, r.z, v.z); v.w = fmaf(ws, r.w, v.w);
       }
@@ -592,7 +608,7 @@ __global__ void moe_combine_kernel(const T* __restrict__ y, const int* __restric
   }
   for (int c = threadIdx.x; c < W; c += blockDim.x) {
     float v = 0.f;
-    for (int s = 0; s < top; ++s) v = fmaf(weight[(size_t)n * top + s], to_float(row_of(s)[c]), v);
+    for (int s = 0; s < top; ++s) v = fmaf(weight ? weight[(size_t)n * top + s] : 1.f, to_float(row_of(s)[c]), v);
     if (shared) v = fmaf(g, to_float(shared[(size_t)n * W + c]), v);
     out[(size_t)n * W + c] = from_float<T>(v);
   }
@@ -607,15 +623,16 @@ GIBBS_EXPORT long gibbs_moe_capacity(int n_pairs, int E, int bm) {
 GIBBS_EXPORT int gibbs_moe_tile(int n_pairs, int E) { return (long)n_pairs <= 64L * E ? 16 : 128; }
 
 // mode 0: the largest logits (+ bias), weights by the softmax over the chosen; mode 1: scores by the softmax over all E
-// outputs, the largest of score + router_bias (a correction that only the choice sees), weights the chosen scores over their sum.
+// outputs, the largest of score + router_bias (a correction that only the choice sees), weights the chosen scores over their sum;
+// mode 2: scores by the sigmoid of every output alone, the largest of score + router_bias, weights the chosen scores.
 GIBBS_EXPORT int gibbs_moe_route_mode(const void* h, long ldh, int dtype, const float* router, const float* router_bias,
                                       const float* shared_gate, int* chosen, float* weight, float* sgate, int n, int W, int E, int top,
                                       int mode, hipStream_t stream) {
-  GIBBS_REQUIRE(mode == 0 || mode == 1, "moe_route: mode %d", mode);
+  GIBBS_REQUIRE(mode >= 0 && mode <= 2, "moe_route: mode %d", mode);
   GIBBS_REQUIRE(h && router && chosen && weight && n > 0 && W > 0 && ldh >= W, "moe_route: bad operands n=%d width=%d", n, W);
   GIBBS_REQUIRE(E > 0 && E <= MOE_MAX_EXPERTS && top > 0 && top <= E, "moe_route: %d of %d experts (at most %d)", top, E, MOE_MAX_EXPERTS);
   GIBBS_REQUIRE(!shared_gate || sgate, "moe_route: a shared expert's gate needs its output");
-  const size_t lds = (size_t)E * sizeof(float) * (mode == 1 ? 2 : 1);
+  const size_t lds = (size_t)E * sizeof(float) * (mode != 0 ? 2 : 1);
   // few rows: a wave per expert (and one for the shared expert's gate) up to 16 waves; many rows fill the chip with 4
   const int threads = n >= 512 ? 256 : WAVE * std::min(16, std::max(4, E + 1));
   if (dtype == GIBBS_F32)
@@ -644,9 +661,16 @@ GIBBS_EXPORT int gibbs_moe_group(const int* chosen, int n_pairs, int E, int bm, 
 // Y[m] = W_a,e X[src(m)] (w_b null), or act(W_a,e X[src(m)]) * (W_b,e X[src(m)]), for every place m of the sorted pairs; e the
 // expert of m's tile; src(m) = pair / top (top > 0: rows of the step, gathered) or m itself (top 0: X is in sorted order).
 // W_a, W_b: [experts, O, I].
+// in_weight [pairs] (null: 1; with w_b only): both products of a place are multiplied by its pair's weight before the activation.
 GIBBS_EXPORT int gibbs_moe_gemm(const void* X, long ldx, int top, const int* sorted_pair, const int* tile_expert, long cap, int bm,
                                 const void* w_a, const void* w_b, void* Y, long ldy, int dtype, int O, int I, int act,
                                 hipStream_t stream) {
+  return gibbs_moe_gemm_weighted(X, ldx, top, sorted_pair, tile_expert, cap, bm, w_a, w_b, nullptr, Y, ldy, dtype, O, I, act, stream);
+}
+GIBBS_EXPORT int gibbs_moe_gemm_weighted(const void* X, long ldx, int top, const int* sorted_pair, const int* tile_expert, long cap, int bm,
+                                         const void* w_a, const void* w_b, const float* in_weight, void* Y, long ldy, int dtype, int O, int I,
+                                         int act, hipStream_t stream) {
+  GIBBS_REQUIRE(!in_weight || w_b, "moe_gemm: weights on the inputs go with the gated products");
   GIBBS_REQUIRE(X && sorted_pair && tile_expert && w_a && Y && O > 0 && I > 0 && ldx >= I && ldy >= O, "moe_gemm: bad operands O=%d I=%d", O, I);
   GIBBS_REQUIRE((bm == 16 || bm == 128) && cap > 0 && cap % bm == 0 && cap / bm <= 65535, "moe_gemm: %ld places in tiles of %d", cap, bm);
   GIBBS_REQUIRE(top >= 0 && act >= 0 && act < ACT_COUNT, "moe_gemm: bad choice count or activation");
@@ -654,7 +678,7 @@ GIBBS_EXPORT int gibbs_moe_gemm(const void* X, long ldx, int top, const int* sor
   const int tiles = (int)(cap / bm);
 #define MOE_PLAIN(T, BM, GLU)                                                                                                     \
   moe_gemm_plain_kernel<T, BM, GLU><<<dim3(ceil_div(O, 64), tiles), 256, 0, stream>>>((const T*)X, ldx, top, sorted_pair, tile_expert, \
-                                                                                     (const T*)w_a, (const T*)w_b, stride, (T*)Y, ldy, O, I, act)
+                                                                                     (const T*)w_a, (const T*)w_b, stride, (T*)Y, ldy, O, I, act, in_weight)
 #define MOE_PLAIN_ANY(T)                                                                  \
   do {                                                                                    \
     if (bm == 128) { if (w_b) MOE_PLAIN(T, 128, true); else MOE_PLAIN(T, 128, false); }    \
@@ -667,15 +691,15 @@ GIBBS_EXPORT int gibbs_moe_gemm(const void* X, long ldx, int top, const int* sor
     if (!aligned) {
       MOE_PLAIN_ANY(bf16);
     } else if (bm == 128) {
-      if (w_b ? launch_tiled<true>((const bf16*)X, ldx, top, sorted_pair, tile_expert, tiles, (const bf16*)w_a, (const bf16*)w_b, stride, (bf16*)Y, ldy, O, I, act, stream)
-              : launch_tiled<false>((const bf16*)X, ldx, top, sorted_pair, tile_expert, tiles, (const bf16*)w_a, nullptr, stride, (bf16*)Y, ldy, O, I, act, stream))
+      if (w_b ? launch_tiled<true>((const bf16*)X, ldx, top, sorted_pair, tile_expert, tiles, (const bf16*)w_a, (const bf16*)w_b, stride, (bf16*)Y, ldy, O, I, act, in_weight, stream)
+              : launch_tiled<false>((const bf16*)X, ldx, top, sorted_pair, tile_expert, tiles, (const bf16*)w_a, nullptr, stride, (bf16*)Y, ldy, O, I, act, nullptr, stream))
         return 1;
     } else if (w_b) {
       moe_gemm_few_kernel<true><<<dim3(ceil_div(O, 32), tiles), 256, 0, stream>>>((const bf16*)X, ldx, top, sorted_pair, tile_expert, (const bf16*)w_a,
-                                                                                 (const bf16*)w_b, stride, (bf16*)Y, ldy, O, I, act);
+                                                                                 (const bf16*)w_b, stride, (bf16*)Y, ldy, O, I, act, in_weight);
     } else {
       moe_gemm_few_kernel<false><<<dim3(ceil_div(O, 32), tiles), 256, 0, stream>>>((const bf16*)X, ldx, top, sorted_pair, tile_expert, (const bf16*)w_a,
-                                                                                  nullptr, stride, (bf16*)Y, ldy, O, I, act);
+                                                                                  nullptr, stride, (bf16*)Y, ldy, O, I, act, nullptr);
     }
   } else {
     return gibbs_fail("moe_gemm: unknown dtype %d", dtype);
@@ -685,7 +709,7 @@ GIBBS_EXPORT int gibbs_moe_gemm(const void* X, long ldx, int top, const int* sor
   GIBBS_LAUNCH_STATUS("moe_gemm");
 }
 
-// out[n] = sum_c weight[n][c] y[pair_pos[n * top + c]] + sgate[n] shared[n]  (shared null: no shared expert; sgate null: 1).
+// out[n] = sum_c weight[n][c] y[pair_pos[n * top + c]] + sgate[n] shared[n]  (shared null: no shared expert; sgate or weight null: 1).
 GIBBS_EXPORT int gibbs_moe_combine(const void* y, const int* pair_pos, const float* weight, const void* shared, const float* sgate,
                                    void* out, int dtype, int n, int top, int W, hipStream_t stream) {
   return gibbs_moe_combine_self(y, pair_pos, weight, shared, sgate, nullptr, out, dtype, n, top, W, stream);
@@ -693,7 +717,7 @@ GIBBS_EXPORT int gibbs_moe_combine(const void* y, const int* pair_pos, const flo
 // self [n, W] (null: none): the rows themselves, which a choice without a place (-1: an identity expert) stands for.
 GIBBS_EXPORT int gibbs_moe_combine_self(const void* y, const int* pair_pos, const float* weight, const void* shared, const float* sgate,
                                         const void* self, void* out, int dtype, int n, int top, int W, hipStream_t stream) {
-  GIBBS_REQUIRE(y && pair_pos && weight && out && n > 0 && top > 0 && W > 0, "moe_combine: bad operands n=%d top=%d width=%d", n, top, W);
+  GIBBS_REQUIRE(y && pair_pos && out && n > 0 && top > 0 && W > 0, "moe_combine: bad operands n=%d top=%d width=%d", n, top, W);
   const size_t bytes = dtype == GIBBS_F32 ? 16 : 8;
   const bool vec = W % 4 == 0 && ((uintptr_t)y % bytes) == 0 && ((uintptr_t)shared % bytes) == 0 && ((uintptr_t)out % bytes) == 0 && ((uintptr_t)self % bytes) == 0;
   const int threads = vec ? (W >= 4096 ? 1024 : (W >= 1024 ? 256 : 64)) : (W >= 1024 ? 256 : 64);

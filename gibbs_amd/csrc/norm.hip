@@ -258,21 +258,33 @@ __global__ void rmsnorm_rows_add_kernel(float* __restrict__ x, const void* __res
 // the scalings: 16-byte accesses, hidden sizes in steps of 4 up to 4 * CHUNKS * blockDim.  Sums, roots and x are float32.
 // MIX: the part's result is itself a weighted sum that no kernel has written yet (a mixture of experts' combination):
 // v = sum_s weight[n][s] * in[place[n][s]] (ascending s, rows of `in` in the activation type) + gate[n] * shared[n]
-// (shared null: none; gate null: 1), float32 throughout.
+// (shared null: none; gate or weight null: 1), float32 throughout.
+// READ: what `out` takes of the new x: READ_NORM its norm (above), READ_ROWS the row as it is (a sublayer that is not normed on
+// its way in), READ_SHIFT the row mixed with the request's previous one, x + (before - x) mu, in a step where every request
+// brings one row: before is the request's state, which the row replaces.
+enum { READ_NORM = 0, READ_ROWS = 1, READ_SHIFT = 2 };
+struct RowShift {
+  const float* mu;        // [hidden]
+  float* state;           // [slots][hidden], slot_stride apart
+  long slot_stride;
+  const int* slot;        // [n]
+};
 struct RowMix {
   const int* place;       // [n, top]
-  const float* weight;    // [n, top]
+  const float* weight;    // [n, top] or null
   const void* shared;     // [n, hidden] or null
   const float* gate;      // [n] or null
   int top;
 };
-template <typename T, int CHUNKS, bool MIX>
+template <typename T, int CHUNKS, bool MIX, int READ>
 __global__ void rows_add_norm_vec_kernel(float* __restrict__ x, const void* __restrict__ in, int parts, size_t part_stride,
                                          const float* __restrict__ gain_d, float eps_d, const float* __restrict__ gain_n, float eps_n,
-                                         T* __restrict__ out, int hidden, RowMix mix) {
+                                         T* __restrict__ out, int hidden, RowMix mix, RowShift shift) {
   __shared__ float scratch[16];
   const size_t at = (size_t)blockIdx.x * hidden;
-  float4 v[CHUNKS], xv[CHUNKS];
+  float4 v[CHUNKS], xv[CHUNKS], before[READ == READ_SHIFT ? CHUNKS : 1];
+  float* st = nullptr;
+  if constexpr (READ == READ_SHIFT) st = shift.state + (size_t)shift.slot[blockIdx.x] * shift.slot_stride;
   float ss = 0.f;
 #pragma unroll
   for (int c = 0; c < CHUNKS; ++c) {
@@ -280,10 +292,11 @@ __global__ void rows_add_norm_vec_kernel(float* __restrict__ x, const void* __re
     v[c] = make_float4(0.f, 0.f, 0.f, 0.f);
     if (i < hidden) {
       xv[c] = *(const float4*)(x + at + i);
+      if constexpr (READ == READ_SHIFT) before[c] = *(const float4*)(st + i);
       if (MIX) {
         const size_t first = (size_t)blockIdx.x * mix.top;
         for (int s = 0; s < mix.top; ++s) {
-          const float w = mix.weight[first + s];
+          const float w = mix.weight ? mix.weight[first + s] : 1.f;
           const float4 r = load4((const T*)in + (size_t)mix.place[first + s] * hidden + i);
           v[c].x = fmaf(w, r.x, v[c].x); v[c].y = fmaf(w, r.y, v[c].y); v[c].z = fmaf(w, r.z, v[c].z); v[c].w = fmaf(w, r.w, v[c].w);
         }
@@ -314,10 +327,17 @@ __global__ void rows_add_norm_vec_kernel(float* __restrict__ x, const void* __re
       if (gain_d) g = *(const float4*)(gain_d + i);
       xv[c].x += v[c].x * scale * g.x; xv[c].y += v[c].y * scale * g.y; xv[c].z += v[c].z * scale * g.z; xv[c].w += v[c].w * scale * g.w;
       *(float4*)(x + at + i) = xv[c];
+      if constexpr (READ == READ_ROWS) store4(out + at + i, xv[c]);
+      if constexpr (READ == READ_SHIFT) {
+        const float4 m = *(const float4*)(shift.mu + i);
+        store4(out + at + i, make_float4(fmaf(before[c].x - xv[c].x, m.x, xv[c].x), fmaf(before[c].y - xv[c].y, m.y, xv[c].y),
+                                         fmaf(before[c].z - xv[c].z, m.z, xv[c].z), fmaf(before[c].w - xv[c].w, m.w, xv[c].w)));
+        *(float4*)(st + i) = xv[c];
+      }
       sx += xv[c].x * xv[c].x + xv[c].y * xv[c].y + xv[c].z * xv[c].z + xv[c].w * xv[c].w;
     }
   }
-  if (!out) return;
+  if (READ != READ_NORM || !out) return;
   sx = block_sum(sx, scratch);
   const float scale_n = 1.0f / sqrtf(sx / (float)hidden + eps_n);
 #pragma unroll
@@ -333,7 +353,8 @@ __global__ void rows_add_norm_vec_kernel(float* __restrict__ x, const void* __re
 
 template <typename T>
 bool launch_rows_add_norm(float* x, const void* in, int parts, long part_stride, const float* gain_d, float eps_d, const float* gain_n,
-                          float eps_n, T* out, int n, int hidden, hipStream_t stream, const RowMix* mixed = nullptr) {
+                          float eps_n, T* out, int n, int hidden, hipStream_t stream, const RowMix* mixed = nullptr, int read = READ_NORM,
+                          const RowShift& shift = RowShift{}) {
   const uintptr_t vec = parts == 1 ? 4 * sizeof(T) : 16;
   if (hidden % 4 || ((uintptr_t)x % 16) || ((uintptr_t)in % vec) || (parts > 1 && part_stride % 4) || (gain_d && ((uintptr_t)gain_d % 16)) ||
       (gain_n && ((uintptr_t)gain_n % 16)) || (out && ((uintptr_t)out % (4 * sizeof(T)))) ||
@@ -342,16 +363,28 @@ bool launch_rows_add_norm(float* x, const void* in, int parts, long part_stride,
   // (few rows: wide workgroups, every load of the row in flight at once)
   const int threads = hidden >= 4096 ? 1024 : (hidden >= 2048 ? 512 : (hidden >= 512 ? 256 : 64));
   const int chunks = ceil_div(hidden, 4 * threads);
-#define GIBBS_ROWS_ADD_NORM(C)                                                                                                              \
-  do {                                                                                                                                      \
-    if (mixed) rows_add_norm_vec_kernel<T, C, true><<<n, threads, 0, stream>>>(x, in, parts, (size_t)part_stride, gain_d, eps_d, gain_n, eps_n, out, hidden, *mixed); \
-    else rows_add_norm_vec_kernel<T, C, false><<<n, threads, 0, stream>>>(x, in, parts, (size_t)part_stride, gain_d, eps_d, gain_n, eps_n, out, hidden, RowMix{}); \
+  if (read == READ_SHIFT && (shift.slot_stride % 4 || ((uintptr_t)shift.state % 16) || ((uintptr_t)shift.mu % 16))) return false;
+  const RowMix mix = mixed ? *mixed : RowMix{};
+#define GIBBS_ROWS_ADD_READ(C, M, R) \
+  rows_add_norm_vec_kernel<T, C, M, R><<<n, threads, 0, stream>>>(x, in, parts, (size_t)part_stride, gain_d, eps_d, gain_n, eps_n, out, hidden, mix, shift)
+#define GIBBS_ROWS_ADD_NORM(C)                                                                     \
+  do {                                                                                             \
+    if (mixed) {                                                                                   \
+      if (read == READ_SHIFT) GIBBS_ROWS_ADD_READ(C, true, READ_SHIFT);                            \
+      else if (read == READ_ROWS) GIBBS_ROWS_ADD_READ(C, true, READ_ROWS);                         \
+      else GIBBS_ROWS_ADD_READ(C, true, READ_NORM);                                                \
+    } else {                                                                                       \
+      if (read == READ_SHIFT) GIBBS_ROWS_ADD_READ(C, false, READ_SHIFT);                           \
+      else if (read == READ_ROWS) GIBBS_ROWS_ADD_READ(C, false, READ_ROWS);                        \
+      else GIBBS_ROWS_ADD_READ(C, false, READ_NORM);                                               \
+    }                                                                                              \
   } while (0)
   if (chunks == 1) GIBBS_ROWS_ADD_NORM(1);
   else if (chunks == 2) GIBBS_ROWS_ADD_NORM(2);
   else if (chunks <= 4) GIBBS_ROWS_ADD_NORM(4);
   else return false;
 #undef GIBBS_ROWS_ADD_NORM
+#undef GIBBS_ROWS_ADD_READ
   return true;
 }
 
@@ -383,6 +416,28 @@ GIBBS_EXPORT int gibbs_rmsnorm_rows_mix_add_norm(float* x, const void* in, const
   else return gibbs_fail("rmsnorm_rows_mix_add_norm: unknown dtype %d", dtype);
   if (!queued) return -1;
   GIBBS_LAUNCH_STATUS("rmsnorm_rows_mix_add_norm");
+}
+
+// x += norm(in) (gain, eps) and what a sublayer that is not normed on its way in reads of the new x: read 0 nothing (out null), 1 its
+// rows, 2 its rows shifted (x + (before - x) mu, before the request's state, which the row replaces: one row per request).  in:
+// [n, hidden] (parts 1) or float32 partial sums, or, with `place`, a mixture of experts' results still to be summed (as above;
+// weight null: 1).  Returns 0, -1 (not queued: sizes or addresses do not allow it) or 1.
+GIBBS_EXPORT int gibbs_rmsnorm_rows_add_read(float* x, const void* in, int parts, long part_stride, const int* place, const float* weight, int top,
+                                             const void* shared, const float* gate, const float* gain, float eps, int read, const float* mu,
+                                             float* state, long slot_stride, const int* slot, void* out, int dtype, int n, int hidden,
+                                             hipStream_t stream) {
+  GIBBS_REQUIRE(x && in && n >= 0 && hidden > 0 && parts >= 1 && (!place || (top >= 1 && parts == 1)), "rmsnorm_rows_add_read: bad sizes n=%d hidden=%d parts=%d", n, hidden, parts);
+  GIBBS_REQUIRE(read >= 0 && read <= 2 && (read == 0 || out) && (read != 2 || (mu && state && slot && slot_stride >= hidden)), "rmsnorm_rows_add_read: bad reader %d", read);
+  if (n == 0) return 0;
+  const RowMix mixed{place, weight, shared, gate, top};
+  const RowShift shift{mu, state, slot_stride, slot};
+  void* o = read ? out : nullptr;
+  bool queued;
+  if (dtype == GIBBS_F32) queued = launch_rows_add_norm<float>(x, in, parts, part_stride, gain, eps, nullptr, 0.f, (float*)o, n, hidden, stream, place ? &mixed : nullptr, read, shift);
+  else if (dtype == GIBBS_BF16) queued = launch_rows_add_norm<bf16>(x, in, parts, part_stride, gain, eps, nullptr, 0.f, (bf16*)o, n, hidden, stream, place ? &mixed : nullptr, read, shift);
+  else return gibbs_fail("rmsnorm_rows_add_read: unknown dtype %d", dtype);
+  if (!queued) return -1;
+  GIBBS_LAUNCH_STATUS("rmsnorm_rows_add_read");
 }
 
 GIBBS_EXPORT int gibbs_rmsnorm_rows_add(float* x, const void* in, int parts, long part_stride, const float* gain, float eps, int dtype,

@@ -392,7 +392,7 @@ int launch_recurrence(const RecurrenceArgs& a, int n_req, hipStream_t stream) {
 }
 
 // ------------------------------------------------------------------------------------------------ a head's read-out, normed and gated
-// y[n, h, :] = o[n, h, :] / sqrt(mean(o^2) + eps) * gain[(h V + j) % gain_len] * act(gate[n, h V + j])
+// y[n, h, :] = o[n, h, :] / sqrt(mean(o^2) + eps) * gain[(h V + j) % gain_len] * act(gate[n, h V + j])    (gate null: no gate)
 template <typename T>
 __global__ __launch_bounds__(64) void head_norm_gate_kernel(const float* __restrict__ o, const float* __restrict__ gain,
                                                             int gain_len, const T* __restrict__ gate, long ld_gate,
@@ -404,7 +404,7 @@ __global__ __launch_bounds__(64) void head_norm_gate_kernel(const float* __restr
   const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)V + eps);
   for (int j = lane; j < V; j += WAVE) {
     const int c = h * V + j;
-    const float g = activate_gate(to_float(gate[(size_t)n * ld_gate + c]), act);
+    const float g = gate ? activate_gate(to_float(gate[(size_t)n * ld_gate + c]), act) : 1.f;
     y[(size_t)n * H * V + c] = from_float<T>(row[j] * inv * gain[c % gain_len] * g);
   }
 }
@@ -557,6 +557,16 @@ GIBBS_EXPORT int gibbs_ssd_rule(const float* q, const float* k, long ldqk, const
   GIBBS_LAUNCH_STATUS("ssd_rule");
 }
 
+// The same with one decay per head and channel, acting on the rows of M, and q, k of every head's own: decay [N, H * D].
+GIBBS_EXPORT int gibbs_gated_outer_rule(const float* q, const float* k, const float* v, const float* decay, float* state, long slot_stride,
+                                        const int* cu, const int* slot, float* out, int n_req, int H, int D, int V, hipStream_t stream) {
+  GIBBS_REQUIRE(q && k && v && decay && state && cu && slot && out, "gated_outer_rule: null operand");
+  if (check_recurrence("gated_outer_rule", n_req, H, H, D, V, slot_stride)) return 1;
+  RecurrenceArgs a{q, k, v, (long)H * D, (long)H * D, (long)H * V, decay, 1, nullptr, nullptr, state, slot_stride, cu, slot, out, H, H, D, V};
+  launch_recurrence<float, RULE_SSD>(a, n_req, stream);
+  GIBBS_LAUNCH_STATUS("gated_outer_rule");
+}
+
 // The gated delta rule over a ragged batch; q, k (unit vectors, q scaled), v, beta, decay float32.
 GIBBS_EXPORT int gibbs_delta_rule(const float* q, const float* k, long ldqk, const float* v, long ldv, const float* beta, const float* decay,
                                   int per_channel, float* state, long slot_stride, const int* cu, const int* slot, float* out,
@@ -582,7 +592,7 @@ GIBBS_EXPORT int gibbs_decayed_outer_rule(const void* r, const void* k, const vo
 
 GIBBS_EXPORT int gibbs_head_norm_gate(const float* o, const float* gain, int gain_len, const void* gate, long ld_gate, void* y,
                                       int dtype, int n_rows, int H, int V, float eps, int act, hipStream_t stream) {
-  GIBBS_REQUIRE(o && gain && gate && y && n_rows > 0 && H > 0 && V > 0 && gain_len > 0 && ld_gate >= (long)H * V && (act == 0 || act == 1),
+  GIBBS_REQUIRE(o && gain && y && n_rows > 0 && H > 0 && V > 0 && gain_len > 0 && (!gate || ld_gate >= (long)H * V) && (act == 0 || act == 1),
                 "head_norm_gate: bad operands rows=%d heads=%d V=%d", n_rows, H, V);
   const dim3 grid(n_rows, H);
   BY_DTYPE(dtype, "head_norm_gate",

@@ -296,6 +296,9 @@ struct NormPart {
   // an RMS norm in groups (1: a plain one) with its gain, for the kernel that norms a result into the stream and the
   // stream for the next sublayer in one pass
   virtual bool group_rms(const float** gain, float* eps, int* groups) const { return false; }
+  // a reader of the stream without a norm: 1 its rows as they are, 2 its rows mixed with the request's previous row (operands
+  // in *mu, *state, *stride); 0: a norm
+  virtual int reader(const float** mu, float** state, long* stride) const { return 0; }
   // a norm that the streams' kernels apply themselves: its kind there (0 root mean square, 1 layer norm) and operands
   virtual bool for_streams(int* kind, const float** gain, const float** bias, float* eps) const { return false; }
 };
@@ -338,7 +341,10 @@ struct Plan {
   bool table_sums() const { return pair_table || pos_table || streams > 1; }
   float embed_scale = 1.0f;            // the table's rows are multiplied by it
   const float* embed_inv_freq = nullptr;   // [hidden / 2]: a sinusoidal position vector is added to the rows
-  bool plain_embedding() const { return embed_scale == 1.0f && !embed_inv_freq && !reinjects && !table_sums(); }
+  bool plain_embedding() const { return embed_scale == 1.0f && !embed_inv_freq && !embed_normed && !reinjects && !table_sums(); }
+  bool embed_normed = false;           // the stream starts as the RMS norm of the table's row
+  const float* embed_gain = nullptr;
+  float embed_eps = 0.f;
   bool reinjects = false;              // the program adds the embedding's output into the stream again
   Matrix head;
   float logit_softcap = 0.f;   // > 0: logits <- cap * tanh(logits / cap)
@@ -503,6 +509,27 @@ struct LayerNorm : NormPart {
   bool for_streams(int* kind, const float** g, const float** b, float* e) const override {
     *kind = 1; *g = gain; *b = bias; *e = eps;
     return true;
+  }
+};
+// What a sublayer that is not normed on its way in reads: the stream's rows in the activation type, or every row mixed with
+// the request's previous one, x + (before - x) mu (the previous row of a request's first one is its state).
+struct StreamRows : NormPart {
+  const float* mu = nullptr;     // [hidden], or null: the rows as they are
+  float* state = nullptr;        // [slots][hidden]
+  long slot_stride = 0;
+  int reader(const float** m, float** st, long* stride) const override {
+    *m = mu; *st = state; *stride = slot_stride;
+    return mu ? 2 : 1;
+  }
+  void* run(Exec& e, float* x, Pending& pending, const int* rows, int n_out) const override {
+    const GibbsStepArgs& a = e.a;
+    const int H = e.p.hidden;
+    if (rows && !e.status) e.status = gibbs_fail("step: the stream is read whole, not by chosen rows");
+    e.settle(x, pending);
+    void* out = e.take((long)n_out * H * e.esize);
+    if (mu) RUN(e, gibbs_stream_shift(x, mu, state, slot_stride, a.row_req, a.cu, a.slot, out, e.p.dtype, a.n_rows, H, a.stream));
+    else RUN(e, gibbs_stream_rows(x, out, e.p.dtype, (long)n_out * H, a.stream));
+    return out;
   }
 };
 struct HostNorm : NormPart {
@@ -1015,7 +1042,8 @@ struct LatentBody : Body {
   const float* sink = nullptr;        // [heads] or null
   const float* inv_freq = nullptr;    // [rot_dims / 2]
   int H = 0, D = 0, R = 0, V = 0, C = 0, q_rank = 0, rot_dims = 0, variant = 0, window = 0;
-  int off_kv = 0, off_g = -1;         // where W_dkv h and the gate start in a projected row (off_g < 0: no gate)
+  // where W_dkv h and the gate start in a projected row (off_kv < 0: the pages are another layer's; off_g < 0: no gate)
+  int off_kv = 0, off_g = -1;
   float scale = 0.f, eps = 0.f;
   void* pages = nullptr;              // [num_pages, 1, page_size, rank + rot]
   int num_pages = 0, page_size = 0, group = 0;
@@ -1040,9 +1068,10 @@ struct LatentBody : Body {
       e.give(cq);
     }
     void* q_lat = e.take((long)N * H * L * e.esize);
-    RUN(e, gibbs_latent_prepare(raw + (long)off_kv * e.esize, in.O, q, ld_q, q_lat, (long)H * L, pages, e.p.dtype, kv_gain, eps, inv_freq,
-                                rot_dims, variant, a.pos, a.row_req, e.table(group), e.width(group), page_size, num_pages, N, H, D, R, C,
-                                a.stream));
+    if (off_kv >= 0 || R > 0)
+      RUN(e, gibbs_latent_prepare(off_kv >= 0 ? raw + (long)off_kv * e.esize : nullptr, in.O, q, ld_q, q_lat, (long)H * L, pages, e.p.dtype, kv_gain, eps,
+                                  inv_freq, rot_dims, variant, a.pos, a.row_req, e.table(group), e.width(group), page_size, num_pages, N, H, D, R, C,
+                                  a.stream));
     RUN(e, gibbs_gemm_heads(q, ld_q, D + R, uk_t, (long)C * D, D, q_lat, (long)H * L, L, e.p.dtype, N, C, D, H, a.stream));
     if (uq.w) e.give(q);
     const PagedAttention t{pages, pages, num_pages, page_size, group, H, 1, L, L, scale, window, nullptr, nullptr, nullptr, 0, sink};
@@ -1057,6 +1086,88 @@ struct LatentBody : Body {
     Pending delta;
     delta.data = e.linear(o, out, N, false, true, true, &delta.parts);
     e.give(o);
+    return delta;
+  }
+};
+
+// ---- differential attention
+// Two softmax maps per head over the same values.  A map is a query head of its own over keys [map 1 | map 2] whose query is zero
+// where the other map's key lies, so the paged attention runs 2 H query heads over G kv heads; then a_1 - lambda a_2 is normed
+// per head, scaled and gated (diff_attention.hip).
+struct DiffAttnBody : Body {
+  Matrix in, out;
+  const float* q_gain = nullptr;
+  const float* k_gain = nullptr;
+  const float* lam = nullptr;
+  const float* inv_freq = nullptr;
+  const float* cos_sin = nullptr;
+  void* kpages = nullptr;
+  void* vpages = nullptr;
+  int H = 0, G = 0, D = 0, V = 0, ks = 0, vs = 0, rot = 0, variant = 0, table_len = 0, window = 0, chunk = 0, gate_off = -1;
+  int num_pages = 0, page_size = 0, group = 0;
+  float scale = 0.f, eps = 0.f, out_scale = 1.f;
+  int cache_group() const override { return group; }
+  Pending general(Exec& e, void* h) const override {
+    const GibbsStepArgs& a = e.a;
+    const int N = a.n_rows;
+    char* raw = (char*)e.linear(h, in, N, false, false, false, nullptr);
+    void* q = e.take((long)N * 2 * H * ks * e.esize);
+    RUN(e, gibbs_diff_prepare(raw, in.O, q, kpages, vpages, e.p.dtype, q_gain, k_gain, eps, inv_freq, rot, variant, cos_sin, table_len, a.pos, a.row_req,
+                              e.table(group), e.width(group), page_size, num_pages, N, H, G, D, V, ks, vs, a.stream));
+    const PagedAttention t{kpages, vpages, num_pages, page_size, group, 2 * H, G, ks, vs, scale, window, nullptr, nullptr, nullptr, 0, nullptr, chunk, 0.f};
+    void* att = attend_prepared(e, t, q, (long)2 * H * ks, (long)2 * H * vs);
+    e.give(q);
+    void* o = e.take((long)N * H * V * e.esize);
+    RUN(e, gibbs_diff_finish(att, vs, gate_off >= 0 ? raw + (long)gate_off * e.esize : nullptr, in.O, lam, eps, out_scale, o, e.p.dtype, N, H, V, a.stream));
+    e.give(att);
+    e.give(raw);
+    Pending delta;
+    delta.data = e.linear(o, out, N, false, true, true, &delta.parts);
+    e.give(o);
+    return delta;
+  }
+};
+
+// ---- gated outer-product recurrence
+// One product gives [a | z | v] of the rows; per head q = silu(a), f = l + (1 - l) sigmoid(z + b), S = diag(f) S + (1 - f) v',
+// read-out S' q normed per head, times a gain, projected back.  A step of one token per request is one kernel between the two
+// products; other steps prepare their rows and walk (gated_outer.hip, recurrent.hip).
+struct GatedOuterBody : Body {
+  Matrix in, out;
+  int H = 0, D = 0, V = 0;
+  const float* bias = nullptr;       // [H D]
+  const float* lower = nullptr;      // [H D]
+  const float* gain = nullptr;       // [V]
+  float* rule_state = nullptr;       // [slots][H][D][V]
+  long slot_stride = 0;
+  float eps = 0.f;
+  Pending general(Exec& e, void* h) const override {
+    const GibbsStepArgs& a = e.a;
+    const int N = a.n_rows;
+    const long C = (long)H * D, HV = (long)H * V;
+    void* raw = e.linear(h, in, N, false, false, false, nullptr);
+    void* y = e.take((long)N * HV * e.esize);
+    if (e.rows_are_requests() && gibbs_gated_outer_step_takes(D, V)) {
+      RUN(e, gibbs_gated_outer_step(raw, in.O, e.p.dtype, bias, lower, gain, eps, rule_state, slot_stride, a.slot, y, a.n_req, H, D, V, a.stream));
+    } else {
+      float* q = (float*)e.take((long)N * C * 4);
+      float* f = (float*)e.take((long)N * C * 4);
+      float* k = (float*)e.take((long)N * C * 4);
+      float* v = (float*)e.take((long)N * HV * 4);
+      RUN(e, gibbs_gated_outer_prep(raw, in.O, e.p.dtype, bias, lower, q, f, k, v, N, H, D, V, a.stream));
+      float* o = (float*)e.take((long)N * HV * 4);
+      RUN(e, gibbs_gated_outer_rule(q, k, v, f, rule_state, slot_stride, a.cu, a.slot, o, a.n_req, H, D, V, a.stream));
+      e.give(q);
+      e.give(f);
+      e.give(k);
+      e.give(v);
+      RUN(e, gibbs_head_norm_gate(o, gain, V, nullptr, 0, y, e.p.dtype, N, H, V, eps, 0, a.stream));
+      e.give(o);
+    }
+    e.give(raw);
+    Pending delta;
+    delta.data = e.linear(y, out, N, false, true, true, &delta.parts);
+    e.give(y);
     return delta;
   }
 };
@@ -1097,7 +1208,9 @@ struct MoeBody : Body {
   const float* shared_gate = nullptr;   // [hidden] float32, or null: the shared expert is added as it is
   // mode 1: scores by a softmax over all router outputs, the choice by score + router_bias, weights the chosen scores over
   // their sum; the router's last `identity` outputs are experts without matrices whose result is the row itself
+  // mode 2: scores by the sigmoid of every output alone, weights the chosen scores as they are
   int mode = 0, identity = 0;
+  bool weigh_input = false;   // the weight multiplies the expert's input (its gate and up products) instead of its result
   Pending general(Exec& e, void* h) const override {
     const int N = e.a.n_rows, W = e.p.hidden, pairs = N * top;
     const int bm = gibbs_moe_tile(pairs, E);
@@ -1112,7 +1225,11 @@ struct MoeBody : Body {
     RUN(e, gibbs_moe_group(chosen, pairs, E, bm, sorted, place, tile_expert, cap, e.a.stream));
     e.give(chosen);
     void* mid = e.take(cap * F * e.esize);
-    RUN(e, gibbs_moe_gemm(h, W, top, sorted, tile_expert, cap, bm, gate, up, mid, F, e.p.dtype, F, W, act, e.a.stream));
+    RUN(e, gibbs_moe_gemm_weighted(h, W, top, sorted, tile_expert, cap, bm, gate, up, weigh_input ? weight : nullptr, mid, F, e.p.dtype, F, W, act, e.a.stream));
+    if (weigh_input) {
+      e.give(weight);
+      weight = nullptr;
+    }
     void* y = e.take(cap * W * e.esize);
     RUN(e, gibbs_moe_gemm(mid, F, 0, sorted, tile_expert, cap, bm, down, nullptr, y, W, e.p.dtype, W, F, 0, e.a.stream));
     e.give(mid);
@@ -1183,6 +1300,10 @@ void Exec::run() {
     RUN(*this, gibbs_embed_tables(p.table, p.pair_table, p.pos_table, p.table_dtype, a.ids, a.pos, a.row_req, a.cu, a.slot, p.prev_state,
                                   p.prev_stride, x, S, N, H, p.vocab, p.buckets, p.mul_prev, p.mul_cur, p.pos_len, a.stream));
     if (p.pair_table) RUN(*this, gibbs_store_last_token(a.ids, a.cu, a.slot, p.prev_state, p.prev_stride, a.n_req, a.stream));
+  } else if (!x && p.embed_normed) {
+    x = (float*)take((long)N * H * 4);
+    mirror = nullptr;
+    RUN(*this, gibbs_embed_norm(p.table, p.table_dtype, a.ids, x, p.embed_gain, p.embed_eps, N, H, p.vocab, a.stream));
   } else if (!x) {
     x = (float*)take((long)N * H * 4);
     mirror = few_rows ? take((long)N * H * 2) : nullptr;
@@ -1247,6 +1368,41 @@ void Exec::run() {
         const float *gain_d = nullptr, *gain_n = nullptr;
         float eps_d = 0.f, eps_n = 0.f;
         Pending& d = deltas[op.value];
+        const float* mu = nullptr;
+        float* shift_state = nullptr;
+        long shift_stride = 0;
+        int reader = next ? p.norms[next->norm]->reader(&mu, &shift_state, &shift_stride) : 0;
+        if (reader && pending.parts == 0 && d.data && p.norms[op.norm]->plain_rms(&gain_d, &eps_d)) {
+          // the same where the next sublayer reads the stream itself: its rows leave in the same pass, or, shifted, where every
+          // request brings one row (elsewhere a row's neighbour is another workgroup's: the reader runs behind this pass)
+          const bool with_rows = reader == 1 || rows_are_requests();
+          if (!with_rows) reader = 0;
+          void* out = with_rows ? take((long)N * H * esize) : nullptr;
+          int fused = -1;
+          const bool mixed = deferred.delta && deferred.delta == d.data;
+          if (!dry && status == 0) {
+            fused = gibbs_rmsnorm_rows_add_read(x, mixed ? deferred.y : d.data, mixed ? 1 : std::max(d.parts, 1), (long)N * H, mixed ? deferred.place : nullptr,
+                                                mixed ? deferred.weight : nullptr, mixed ? deferred.top : 0, mixed ? deferred.shared : nullptr,
+                                                mixed ? deferred.gate : nullptr, gain_d, eps_d, reader, mu, shift_state, shift_stride, a.slot, out, p.dtype, N, H,
+                                                a.stream);
+            if (fused > 0) status = 1;
+          } else if (H % 4 == 0 && H <= 16384) {
+            fused = 0;      // (a dry run: the same buffers as the real one will take)
+          }
+          if (fused == 0) {
+            if (mixed) mix_done();
+            give(d.data);
+            d = Pending{};
+            give(mirror);
+            mirror = nullptr;
+            if (with_rows) {
+              rows[next->result] = out;
+              ++i;
+            }
+            break;
+          }
+          give(out);
+        }
         if (next && pending.parts == 0 && d.data && p.norms[op.norm]->plain_rms(&gain_d, &eps_d) && p.norms[next->norm]->plain_rms(&gain_n, &eps_n)) {
           void* out = take((long)N * H * esize);
           int fused = -1;
@@ -1378,6 +1534,8 @@ int check_args(const Plan* p, const GibbsStepArgs* a, bool whole_step) {
   }
   GIBBS_REQUIRE(!p->table_sums() || (p->embed_scale == 1.0f && !p->embed_inv_freq && !p->reinjects), "step: an embedding with a pair or position table, or several streams, takes no scale, sinusoid or second addition");
   GIBBS_REQUIRE(!a->x_in || !p->table_sums() || a->n_ops, "step: this model's embedding is more than the token table's rows: the step embeds its rows itself");
+  GIBBS_REQUIRE(!p->embed_normed || (p->embed_scale == 1.0f && !p->embed_inv_freq && !p->reinjects && !p->table_sums()), "step: a normed embedding takes no scale, sinusoid, second addition or further tables");
+  GIBBS_REQUIRE(!a->x_in || !p->embed_normed || a->n_ops, "step: this model's embedding is normed: the step embeds its rows itself");
   GIBBS_REQUIRE(!p->pair_table || (p->prev_state && a->slot && a->cu && a->row_req), "step: the pair table needs the requests' slots");
   const int first = a->n_ops ? a->first_op : 0, last = a->n_ops ? a->first_op + a->n_ops : (int)p->ops.size();
   for (int i = first; i < last; ++i) {
@@ -1512,7 +1670,7 @@ GIBBS_EXPORT int gibbs_plan_body_latent(void* plan, const GibbsLatentSpec* d) {
   Plan* p = open_plan(plan);
   if (!p) return -1;
   if (!d || !(d->w_in && d->w_out && d->w_uk_t && d->w_uv && d->pages && d->heads > 0 && d->dim > 0 && d->rot >= 0 && d->vdim > 0 &&
-              d->rank > 0 && d->in_rows > 0 && d->off_kv >= 0 && d->off_kv + d->rank + d->rot <= d->in_rows && d->num_pages > 0 &&
+              d->rank > 0 && d->in_rows > 0 && (d->off_kv < 0 || (d->kv_gain && d->off_kv + d->rank + d->rot <= d->in_rows)) && d->num_pages > 0 &&
               d->page_size > 0 && d->group >= 0 && d->window >= 0 && (d->rot_dims == 0 || d->inv_freq) && d->rot_dims <= d->rot &&
               (!d->w_uq || d->q_rank > 0) && (d->off_g < 0 || d->off_g + d->heads * d->vdim <= d->in_rows))) {
     gibbs_fail("plan: bad latent attention");
@@ -1529,6 +1687,74 @@ GIBBS_EXPORT int gibbs_plan_body_latent(void* plan, const GibbsLatentSpec* d) {
   b->pages = d->pages; b->num_pages = d->num_pages; b->page_size = d->page_size; b->group = d->group;
   p->bodies.push_back(std::move(b));
   return (int)p->bodies.size() - 1;
+}
+
+GIBBS_EXPORT int gibbs_plan_body_diff_attention(void* plan, const GibbsDiffAttentionSpec* d) {
+  Plan* p = open_plan(plan);
+  if (!p) return -1;
+  if (!d || !(d->w_in && d->w_out && d->q_gain && d->k_gain && d->lam && d->kpages && d->vpages && d->heads > 0 && d->kv_heads > 0 &&
+              d->heads % d->kv_heads == 0 && d->dim > 0 && d->vdim > 0 && d->k_stored >= 2 * d->dim && d->v_stored >= d->vdim && d->k_stored <= 512 &&
+              d->v_stored <= 512 && d->num_pages > 0 && d->page_size > 0 && d->group >= 0 && d->window >= 0 && d->chunk >= 0 && !(d->window && d->chunk) &&
+              (!d->inv_freq || (d->rot > 0 && d->rot % 2 == 0 && d->rot <= d->dim)))) {
+    gibbs_fail("plan: bad differential attention");
+    return -1;
+  }
+  const int used = 2 * (d->heads + d->kv_heads) * d->dim + d->kv_heads * d->vdim;
+  if (d->in_rows < used || (d->gate_off >= 0 && (d->gate_off < used || d->gate_off + d->heads > d->in_rows))) {
+    gibbs_fail("plan: a projection of %d rows is too short for the differential attention", d->in_rows);
+    return -1;
+  }
+  auto b = std::make_unique<DiffAttnBody>();
+  b->in = Matrix{d->w_in, nullptr, d->in_rows, p->hidden};
+  b->out = Matrix{d->w_out, nullptr, p->hidden, d->heads * d->vdim};
+  b->q_gain = d->q_gain; b->k_gain = d->k_gain; b->lam = d->lam; b->inv_freq = d->inv_freq; b->cos_sin = d->cos_sin;
+  b->kpages = d->kpages; b->vpages = d->vpages;
+  b->H = d->heads; b->G = d->kv_heads; b->D = d->dim; b->V = d->vdim; b->ks = d->k_stored; b->vs = d->v_stored;
+  b->rot = d->inv_freq ? d->rot : 0; b->variant = d->variant; b->table_len = d->cos_sin ? d->table_len : 0;
+  b->window = d->window; b->chunk = d->chunk; b->gate_off = d->gate_off;
+  b->num_pages = d->num_pages; b->page_size = d->page_size; b->group = d->group;
+  b->scale = d->scale; b->eps = d->eps; b->out_scale = d->out_scale;
+  p->bodies.push_back(std::move(b));
+  return (int)p->bodies.size() - 1;
+}
+
+GIBBS_EXPORT int gibbs_plan_body_gated_outer(void* plan, const GibbsGatedOuterSpec* d) {
+  Plan* p = open_plan(plan);
+  if (!p) return -1;
+  if (!d || !(d->w_in && d->w_out && d->f_bias && d->lower && d->gain && d->rule_state && d->heads > 0 && d->heads <= 65535 && d->dim > 0 &&
+              d->dim <= 256 && d->vdim > 0 && d->slot_stride >= (long)d->heads * d->dim * d->vdim)) {
+    gibbs_fail("plan: bad gated outer-product mixer");
+    return -1;
+  }
+  auto b = std::make_unique<GatedOuterBody>();
+  b->in = Matrix{d->w_in, nullptr, d->heads * (2 * d->dim + d->vdim), p->hidden};
+  b->out = Matrix{d->w_out, nullptr, p->hidden, d->heads * d->vdim};
+  b->H = d->heads; b->D = d->dim; b->V = d->vdim; b->bias = d->f_bias; b->lower = d->lower; b->gain = d->gain;
+  b->rule_state = d->rule_state; b->slot_stride = d->slot_stride; b->eps = d->eps;
+  p->bodies.push_back(std::move(b));
+  return (int)p->bodies.size() - 1;
+}
+
+GIBBS_EXPORT int gibbs_plan_embedding_norm(void* plan, const float* gain, float eps) {
+  Plan* p = open_plan(plan);
+  if (!p) return -1;
+  p->embed_normed = true; p->embed_gain = gain; p->embed_eps = eps;
+  return 0;
+}
+GIBBS_EXPORT int gibbs_plan_stream_rows(void* plan) {
+  Plan* p = open_plan(plan);
+  if (!p) return -1;
+  p->norms.push_back(std::make_unique<StreamRows>());
+  return (int)p->norms.size() - 1;
+}
+GIBBS_EXPORT int gibbs_plan_shifted_rows(void* plan, const float* mu, float* state, long slot_stride) {
+  Plan* p = open_plan(plan);
+  if (!p) return -1;
+  if (!(mu && state && slot_stride >= p->hidden)) { gibbs_fail("plan: bad shift by one token"); return -1; }
+  auto n = std::make_unique<StreamRows>();
+  n->mu = mu; n->state = state; n->slot_stride = slot_stride;
+  p->norms.push_back(std::move(n));
+  return (int)p->norms.size() - 1;
 }
 
 GIBBS_EXPORT int gibbs_plan_body_mlp(void* plan, const void* w_up, const void* w_down, int F, const float* coef, float eps) {
@@ -1688,8 +1914,17 @@ GIBBS_EXPORT int gibbs_plan_moe_scores(void* plan, int body, int mode, int ident
   Plan* p = open_plan(plan);
   if (!p) return -1;
   MoeBody* m = p->has_body(body) ? dynamic_cast<MoeBody*>(p->bodies[body].get()) : nullptr;
-  if (!m || (mode != 0 && mode != 1) || identity < 0 || m->E + identity > 1024 || m->top > m->E + identity) { gibbs_fail("plan: body %d is no mixture of experts, or bad router options", body); return -1; }
+  if (!m || mode < 0 || mode > 2 || identity < 0 || m->E + identity > 1024 || m->top > m->E + identity) { gibbs_fail("plan: body %d is no mixture of experts, or bad router options", body); return -1; }
   m->mode = mode; m->identity = identity;
+  return 0;
+}
+
+GIBBS_EXPORT int gibbs_plan_moe_weigh_input(void* plan, int body) {
+  Plan* p = open_plan(plan);
+  if (!p) return -1;
+  MoeBody* m = p->has_body(body) ? dynamic_cast<MoeBody*>(p->bodies[body].get()) : nullptr;
+  if (!m || m->identity > 0 || m->shared_gate_up.w) { gibbs_fail("plan: body %d is no mixture of experts, or has shared or identity experts", body); return -1; }
+  m->weigh_input = true;
   return 0;
 }
 

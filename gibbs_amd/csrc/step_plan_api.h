@@ -161,15 +161,50 @@ int gibbs_plan_logit_softcap(void* plan, float cap);
 // A mixture of experts' router: mode 0 as described above; mode 1: scores s = softmax over all router outputs, the `top`
 // largest of s + router_bias are chosen, their weights are their scores s over the sum of those (+ 1e-20).  The router
 // then has experts + identity outputs, the last `identity` of which are experts without matrices that return their input.
+// mode 2: scores s = sigmoid of every output alone, the `top` largest of s + router_bias (null: of the logits), weights their s.
 int gibbs_plan_moe_scores(void* plan, int body, int mode, int identity);
+// The choices' weights go in with the row: the result is the sum of expert(weight * h) (no shared or identity experts).
+int gibbs_plan_moe_weigh_input(void* plan, int body);
+
+// The stream starts as the RMS norm of the token table's row, times gain (null: 1).
+int gibbs_plan_embedding_norm(void* plan, const float* gain, float eps);
+// Readers of the stream, to be used where a norm is: its rows as they are, in the activation type; and its rows mixed with the
+// request's previous row, x + (before - x) mu (mu [hidden]; state [slots][hidden] float32: the requests' last rows, zeros at a
+// sequence's start).
+int gibbs_plan_stream_rows(void* plan);
+int gibbs_plan_shifted_rows(void* plan, const float* mu, float* state, long slot_stride);
+// Gated outer-product mixer: w_in [heads * (2 dim + vdim), hidden], rows [a | z | v]; per head q = silu(a), f = lower +
+// (1 - lower) sigmoid(z + f_bias) (both [heads * dim]), S = diag(f) S + (1 - f) v', read-out S' q divided by its root mean
+// square, times gain [vdim].  rule_state [slots][heads][dim][vdim] float32.
+struct GibbsGatedOuterSpec {
+  const void* w_in; const void* w_out;
+  const float* f_bias; const float* lower; const float* gain;
+  float* rule_state; long slot_stride;
+  int heads, dim, vdim;
+  float eps;
+};
+int gibbs_plan_body_gated_outer(void* plan, const struct GibbsGatedOuterSpec* spec);
+// Differential attention: w_in [in_rows, hidden], rows [q: heads x 2 maps x dim | k: kv_heads x 2 maps x dim | v: kv_heads x
+// vdim | at gate_off (< 0: none) one gate per head]; every map normed (q_gain, k_gain [dim], eps) and its first `rot` entries
+// turned; two softmax maps per head over the same values, a_1 - lam a_2 (lam: one float32 on the device) divided by its root
+// mean square, times out_scale, times sigmoid(gate).  Pages: keys [num_pages, kv_heads, page_size, k_stored >= 2 dim], values
+// [.., v_stored >= vdim].  chunk > 0: a row sees its own stretch of `chunk` positions; window > 0: the last `window`.
+struct GibbsDiffAttentionSpec {
+  const void* w_in; const void* w_out;
+  const float* q_gain; const float* k_gain; const float* lam; const float* inv_freq; const float* cos_sin;
+  void* kpages; void* vpages;
+  int in_rows, heads, kv_heads, dim, vdim, k_stored, v_stored, rot, variant, table_len, window, chunk, gate_off, num_pages, page_size, group;
+  float scale, eps, out_scale;
+};
+int gibbs_plan_body_diff_attention(void* plan, const struct GibbsDiffAttentionSpec* spec);
 
 // Layer norm with gain and bias (either may be null: 1 and 0).
 int gibbs_plan_norm_layer(void* plan, const float* gain, const float* bias, float eps);
 
 // Latent attention: one cached row [latent (rank) | rotated key part (rot)] per token, shared by all heads.  w_in
 // [in_rows, hidden]: the rows of the queries (heads * (dim + rot); or, with w_uq [heads * (dim + rot), q_rank], the q_rank
-// rows of the queries' own latent, which is RMS-normed with q_gain), at off_kv the rank + rot rows of the keys' and values'
-// down-projection (the first rank RMS-normed with kv_gain), at off_g (< 0: none) the heads * vdim rows of a sigmoid gate on
+// rows of the queries' own latent, which is RMS-normed with q_gain), at off_kv (< 0: none, the pages are another layer's and are
+// only read) the rank + rot rows of the keys' and values' down-projection (the first rank RMS-normed with kv_gain), at off_g (< 0: none) the heads * vdim rows of a sigmoid gate on
 // the heads' outputs.  w_uk_t [heads, rank, dim]: every head's key up-projection, transposed; w_uv [heads * vdim, rank].
 // A query head is [dim unrotated | rot rotated]; the first rot_dims entries of a rotated part turn with the position
 // (variant 0: pairs (i, i + rot_dims / 2), 1: pairs (2 i, 2 i + 1); inv_freq [rot_dims / 2]).  window 0: all keys;

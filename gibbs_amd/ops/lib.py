@@ -86,6 +86,22 @@ _SIGNATURES = {
                                c_int, c_void_p],
     "gibbs_causal_conv": [c_void_p, c_long, c_int, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_long,
                           c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
+    "gibbs_embed_norm": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_float, c_int, c_int, c_int, c_void_p],
+    "gibbs_stream_rows": [c_void_p, c_void_p, c_int, c_long, c_void_p],
+    "gibbs_stream_shift": [c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p],
+    "gibbs_rmsnorm_rows_add_read": [c_void_p, c_void_p, c_int, c_long, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_float, c_int,
+                                    c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p],
+    "gibbs_diff_prepare": [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_float, c_void_p, c_int, c_int, c_void_p,
+                           c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
+    "gibbs_diff_finish": [c_void_p, c_int, c_void_p, c_long, c_void_p, c_float, c_float, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
+    "gibbs_gated_outer_prep": [c_void_p, c_long, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
+                               c_void_p],
+    "gibbs_gated_outer_step": [c_void_p, c_long, c_int, c_void_p, c_void_p, c_void_p, c_float, c_void_p, c_long, c_void_p, c_void_p, c_int, c_int,
+                               c_int, c_int, c_void_p],
+    "gibbs_gated_outer_rule": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
+                               c_void_p],
+    "gibbs_moe_gemm_weighted": [c_void_p, c_long, c_int, c_void_p, c_void_p, c_long, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_int,
+                                c_int, c_int, c_int, c_void_p],
     "gibbs_ssd_prep": [c_void_p, c_long, c_void_p, c_long, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p],
     "gibbs_ssd_step": [c_void_p, c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int,
                        c_void_p],

@@ -148,6 +148,44 @@ class SandwichBlock(Block):
             plan.add_normed(after.emit(plan), delta)
 
 
+@register_arrangement("post_norm")
+class PostNormBlock(Block):
+    """Sublayers that read the stream itself and are normed on their way back into it:
+
+        x = x + norm1(mixer(x));   x = x + norm2(ffn(x))
+
+    Roles: `mixer`, `norm1`, and optionally `ffn` with `norm2` (a layer without a feed-forward), and optionally `mixer_input`: a
+    part with state of its own (kind `token_shift`) that makes the rows the mixer reads from the stream.  Norms may carry a scale
+    per channel (`NormSpec.scale`).  The norm of a sublayer's result, its addition into the float32 stream and the rows that
+    the next sublayer reads are one pass where the step's shape allows it (csrc/step_plan.hip)."""
+
+    def __init__(self, spec, hidden, layer_index):
+        super().__init__(spec, hidden, layer_index)
+        self.has_ffn = "ffn" in self.named
+        missing = [r for r in ["mixer", "norm1"] + (["norm2"] if self.has_ffn else []) if r not in self.named]
+        if missing:
+            raise ValueError(f"layer {spec.name!r} lacks the parts {missing}")
+
+    def bind(self, weights, rt: Runtime) -> None:
+        super().bind(weights, rt)
+        if rt.act_dtype == torch.bfloat16:       # (tile-ordered copies for the few-row products of decode steps)
+            self.mixer.pack_matrices()
+            if self.has_ffn:
+                self.ffn.pack_matrices()
+
+    def emit(self, plan, caches) -> None:
+        through = self.named.get("mixer_input")
+        reader = plan.stream_rows() if through is None else through.emit(plan, caches["mixer_input"])
+        subs = [(reader, self.mixer.emit(plan, caches["mixer"]), self.norm1)]
+        if self.has_ffn:
+            subs.append((plan.stream_rows(), self.ffn.emit(plan), self.norm2))
+        for reader, body, after in subs:
+            h = plan.normed(reader)
+            delta = plan.apply(body, h)
+            plan.drop(h)
+            plan.add_normed(after.emit(plan), delta)
+
+
 @register_connection("hyper")
 class HyperConnection(Connection):
     """A sublayer over S residual streams x_1 .. x_S: it reads u = sum_s in[s] x_s and, with its result y, writes all

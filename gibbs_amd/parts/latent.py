@@ -12,6 +12,8 @@ With h the mixer's input, H heads, per head `dim` unrotated and `rot_dim` rotate
               exponential joins the denominator, with no key and no value
     output    the heads' results, optionally times sigmoid(W_g h) (`gate`), through W_o
 
+A mixer whose params name `kv_source` has no W_dkv: it reads that layer's cached rows with its own queries, W_uk and W_uv.
+
 Only [c | rotate(k_r)] is cached: one row of kv_rank + rot_dim values per token and layer, whatever the number of
 heads.  The kernels work on those rows directly: since q_i . W_uk,i c = (W_uk,i' q_i) . c, every head's query becomes
 [W_uk,i' q_i | rotate(q_r,i)] and all heads attend over the same cached rows (one kv head whose values are the rows
@@ -44,6 +46,7 @@ class LatentAttentionMixer(Mixer):
         self.window = None if p.get("window") is None else int(p["window"])
         self.sink, self.gate = bool(p.get("sink", False)), bool(p.get("gate", False))
         self.norm_eps = float(p["norm_eps"])
+        self.source = p.get("kv_source")
         if self.window is not None and self.window <= 0:
             raise ValueError(f"attention window {self.window} must be positive")
         if min(self.heads, self.dim, self.vdim, self.kv_rank) <= 0 or self.rot_dim < 0:
@@ -53,7 +56,12 @@ class LatentAttentionMixer(Mixer):
         self.position = build_position(spec.position, self.rot_dim) if self.rot_dim > 0 else None
 
     # ------------------------------------------------------------------ what it asks for
+    def kv_source(self) -> Optional[int]:
+        return self.source
+
     def cache_need(self) -> Optional[CacheNeed]:
+        if self.source is not None:
+            return None
         # one "kv head" whose keys are the cached rows; the values are read from the same rows (no pages of their own)
         return CacheNeed(1, self.kv_rank + self.rot_dim, self.window, 0)
 
@@ -63,9 +71,10 @@ class LatentAttentionMixer(Mixer):
     def tensor_decls(self) -> List[TensorDecl]:
         t, W, H = self.spec.tensors, self.hidden, self.heads
         qk = H * (self.dim + self.rot_dim)
-        decls = [TensorDecl(t["dkv"], (self.kv_rank + self.rot_dim, W)), TensorDecl(t["dkv_norm"], (self.kv_rank,), FLOAT32, init="gain"),
-                 TensorDecl(t["uk"], (H * self.dim, self.kv_rank)), TensorDecl(t["uv"], (H * self.vdim, self.kv_rank)),
+        decls = [TensorDecl(t["uk"], (H * self.dim, self.kv_rank)), TensorDecl(t["uv"], (H * self.vdim, self.kv_rank)),
                  TensorDecl(t["o"], (W, H * self.vdim))]
+        if self.source is None:
+            decls += [TensorDecl(t["dkv"], (self.kv_rank + self.rot_dim, W)), TensorDecl(t["dkv_norm"], (self.kv_rank,), FLOAT32, init="gain")]
         if self.q_rank:
             decls += [TensorDecl(t["dq"], (self.q_rank, W)), TensorDecl(t["dq_norm"], (self.q_rank,), FLOAT32, init="gain"),
                       TensorDecl(t["uq"], (qk, self.q_rank))]
@@ -82,7 +91,9 @@ class LatentAttentionMixer(Mixer):
         t = self.spec.tensors
         # one product for everything that reads the normed rows: [W_dq or W_q | W_dkv | W_g], every segment starting at
         # a multiple of 8 rows (zero rows between), so that slices of the result stay 16-byte aligned
-        segments = [weights[t["dq"]] if self.q_rank else weights[t["q"]], weights[t["dkv"]]]
+        segments = [weights[t["dq"]] if self.q_rank else weights[t["q"]]]
+        if self.source is None:
+            segments.append(weights[t["dkv"]])
         if self.gate:
             segments.append(weights[t["g"]])
         rows, offsets = [], []
@@ -93,8 +104,8 @@ class LatentAttentionMixer(Mixer):
             if pad:
                 rows.append(torch.zeros((pad, seg.shape[1]), dtype=seg.dtype, device=seg.device))
         self.w_in = torch.cat(rows, dim=0).contiguous()
-        self.off_kv = offsets[1]
-        self.off_g = offsets[2] if self.gate else -1
+        self.off_kv = offsets[1] if self.source is None else -1
+        self.off_g = offsets[-1] if self.gate else -1
         self.w_uq = weights[t["uq"]] if self.q_rank else None
         self.q_gain = weights[t["dq_norm"]] if self.q_rank else None
         if self.q_rank and rt.act_dtype == torch.bfloat16 and rt.fold_gains:
@@ -102,7 +113,7 @@ class LatentAttentionMixer(Mixer):
             # norms' gains of the other models do), and steps of few rows take the product that norms its rows itself
             self.w_uq = (self.w_uq.float() * self.q_gain[None, :]).to(self.w_uq.dtype)
             self.q_gain = None
-        self.kv_gain = weights[t["dkv_norm"]]
+        self.kv_gain = weights[t["dkv_norm"]] if self.source is None else None
         # every head's key up-projection transposed, [heads, kv_rank, dim]: the product that takes a head's unrotated
         # query part to the latent's size reads it as a matrix [out, in]
         self.w_uk_t = weights[t["uk"]].view(self.heads, self.dim, self.kv_rank).transpose(1, 2).contiguous()
@@ -122,7 +133,8 @@ class LatentAttentionMixer(Mixer):
     def product_shapes(self):
         H, W = self.heads, self.hidden
         qk = H * (self.dim + self.rot_dim)
-        shapes = [((self.q_rank or qk) + self.kv_rank + self.rot_dim + (H * self.vdim if self.gate else 0), W), (W, H * self.vdim)]
+        kv = self.kv_rank + self.rot_dim if self.source is None else 0
+        shapes = [((self.q_rank or qk) + kv + (H * self.vdim if self.gate else 0), W), (W, H * self.vdim)]
         if self.q_rank:
             shapes.append((qk, self.q_rank))
         shapes += [(H * self.kv_rank, self.dim), (H * self.vdim, self.kv_rank)]     # per head: flops of [kv_rank, dim] and [vdim, kv_rank]

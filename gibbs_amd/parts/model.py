@@ -26,6 +26,7 @@ class DecoderModel(Part):
         self.spec = spec
         self.blocks: List[Block] = [build_block(ls, spec.hidden, i) for i, ls in enumerate(spec.layers)]
         self.final_norm = build_norm(spec.final_norm, spec.hidden)
+        self.embedding_norm = build_norm(spec.embedding_norm, spec.hidden) if spec.embedding_norm is not None else None
         if any(not 0 < r < len(spec.order) for r in spec.reinject_before):
             raise ValueError(f"the embedding's output is added again before runs {list(spec.reinject_before)}; the order has {len(spec.order)}")
         for i in spec.order:
@@ -50,6 +51,8 @@ class DecoderModel(Part):
     def tensor_decls(self) -> List[TensorDecl]:
         s = self.spec
         decls = [TensorDecl(s.embedding, (s.vocab, s.hidden))]
+        if self.embedding_norm is not None:
+            decls += self.embedding_norm.tensor_decls()
         decls += self.final_norm.tensor_decls()
         for b in self.blocks:
             decls += b.tensor_decls()
@@ -128,5 +131,7 @@ class DecoderModel(Part):
         if streams - {self.spec.streams} or (self.spec.streams != 1 and len(streams) != 1):
             raise ValueError(f"the model has {self.spec.streams} residual streams, its layers are connected for {sorted(streams)}")
         self.final_norm.bind(weights, rt)
+        if self.embedding_norm is not None:
+            self.embedding_norm.bind(weights, rt)
         for b in self.blocks:
             b.bind(weights, rt)

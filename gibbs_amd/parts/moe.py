@@ -11,6 +11,11 @@ s + correction (tensor `correction`, one number per output, seen by the choice a
 divided by their sum (+ 1e-20).  `identity: n`: the router has `experts + n` outputs, and the last n of them are experts
 without matrices whose result is the row itself.  `shared.gate: False` adds the shared expert as it is.
 
+`scores: "sigmoid"` is a third router: scores s = sigmoid(z), the `top` largest of s + correction (without a correction: the
+largest z), weights the chosen experts' s as they are.  `weigh: "input"` puts a choice's weight on the expert's input instead
+of its output: the row's result is the sum of expert(weight * h) (the weight multiplies the gate and up products' float32
+sums before the activation: they have no biases).
+
 The experts' matrices are kept stacked, [experts, F, hidden] and [experts, hidden, F]: the step sorts its (row,
 choice) pairs by expert on the device and runs the experts' products over tiles of pairs (csrc/moe.hip), so the
 host never learns which experts a step uses."""
@@ -36,9 +41,12 @@ class MoeFeedForward(FeedForward):
         self.scores = p.get("scores", "softmax_top")
         self.identity = int(p.get("identity", 0))
         self.outputs = self.experts + self.identity         # rows of the router
-        if self.scores not in ("softmax_top", "softmax_all") or self.identity < 0:
-            raise ValueError(f"router scores {self.scores!r} ('softmax_top' or 'softmax_all') with {self.identity} identity experts")
-        if self.scores == "softmax_all":
+        if self.scores not in ops.MOE_SCORES or self.identity < 0:
+            raise ValueError(f"router scores {self.scores!r} (one of {sorted(ops.MOE_SCORES)}) with {self.identity} identity experts")
+        self.weigh = p.get("weigh", "output")
+        if self.weigh not in ("output", "input") or (self.weigh == "input" and (self.identity or p.get("shared"))):
+            raise ValueError(f"weights on an expert's {self.weigh!r} ('output', or 'input' without identity or shared experts)")
+        if self.scores != "softmax_top":
             self.router_bias_name = spec.tensors.get("correction")
         shared = p.get("shared")
         self.shared_inter = int(shared["inter"]) if shared else 0

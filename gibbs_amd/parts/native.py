@@ -69,6 +69,22 @@ class SsdSpec(ctypes.Structure):
                 ("taps_per_channel", c_int), ("norm_groups", c_int), ("eps", ctypes.c_float)]
 
 
+class GatedOuterSpec(ctypes.Structure):
+    """GibbsGatedOuterSpec of csrc/step_plan_api.h."""
+    _fields_ = [("w_in", c_void_p), ("w_out", c_void_p), ("f_bias", c_void_p), ("lower", c_void_p), ("gain", c_void_p),
+                ("rule_state", c_void_p), ("slot_stride", c_long), ("heads", c_int), ("dim", c_int), ("vdim", c_int), ("eps", ctypes.c_float)]
+
+
+class DiffAttentionSpec(ctypes.Structure):
+    """GibbsDiffAttentionSpec of csrc/step_plan_api.h."""
+    _fields_ = [("w_in", c_void_p), ("w_out", c_void_p), ("q_gain", c_void_p), ("k_gain", c_void_p), ("lam", c_void_p), ("inv_freq", c_void_p),
+                ("cos_sin", c_void_p), ("kpages", c_void_p), ("vpages", c_void_p),
+                ("in_rows", c_int), ("heads", c_int), ("kv_heads", c_int), ("dim", c_int), ("vdim", c_int), ("k_stored", c_int), ("v_stored", c_int),
+                ("rot", c_int), ("variant", c_int), ("table_len", c_int), ("window", c_int), ("chunk", c_int), ("gate_off", c_int),
+                ("num_pages", c_int), ("page_size", c_int), ("group", c_int),
+                ("scale", ctypes.c_float), ("eps", ctypes.c_float), ("out_scale", ctypes.c_float)]
+
+
 class MoeSpec(ctypes.Structure):
     """GibbsMoeSpec of csrc/step_plan_api.h."""
     _fields_ = [("router", c_void_p), ("router_bias", c_void_p), ("gate", c_void_p), ("up", c_void_p), ("down", c_void_p),
@@ -112,6 +128,12 @@ def declare(lib) -> None:
         "gibbs_plan_body_ssd": ([P, POINTER(SsdSpec)], I),
         "gibbs_plan_logit_softcap": ([P, F], I),
         "gibbs_plan_moe_scores": ([P, I, I, I], I),
+        "gibbs_plan_moe_weigh_input": ([P, I], I),
+        "gibbs_plan_embedding_norm": ([P, P, F], I),
+        "gibbs_plan_stream_rows": ([P], I),
+        "gibbs_plan_shifted_rows": ([P, P, P, LG], I),
+        "gibbs_plan_body_gated_outer": ([P, POINTER(GatedOuterSpec)], I),
+        "gibbs_plan_body_diff_attention": ([P, POINTER(DiffAttentionSpec)], I),
         "gibbs_plan_op_rows": ([P, I, I], I),
         "gibbs_plan_body_latent": ([P, POINTER(LatentSpec)], I),
         "gibbs_plan_body_mlp": ([P, P, P, I, P, F], I),
@@ -326,6 +348,54 @@ class NativePlan:
         d.eps = m.norm_eps
         return self._made(L.library().gibbs_plan_body_ssd(self.handle, ctypes.byref(d)))
 
+    def embedding_norm(self, gain: Optional[torch.Tensor], eps: float) -> None:
+        """The stream starts as the RMS norm of the table's row (times `gain`)."""
+        (g,) = self._held(gain)
+        self._made(L.library().gibbs_plan_embedding_norm(self.handle, g, float(eps)))
+        self.plain_embedding = False
+
+    def stream_rows(self) -> int:
+        """A reader of the stream (used as a norm's number): its rows as they are, in the activation type."""
+        return self._made(L.library().gibbs_plan_stream_rows(self.handle))
+
+    def shifted_rows(self, *, mu: torch.Tensor, state: torch.Tensor) -> int:
+        """A reader of the stream: every row mixed with the one before it, x + (x' - x) mu; state float32 [slots, hidden] in
+        the arena: the requests' last rows."""
+        assert mu.dtype == torch.float32 and mu.is_contiguous() and state.dtype == torch.float32 and state.stride(1) == 1
+        (m,) = self._held(mu)
+        self.keep.append(state)
+        return self._made(L.library().gibbs_plan_shifted_rows(self.handle, m, state.data_ptr(), int(state.stride(0))))
+
+    def gated_outer(self, m, *, rule_state: torch.Tensor) -> int:
+        """The gated outer-product mixer `m` (parts/gated_outer.py) over its state [slots, heads, dim, vdim] in the arena."""
+        assert rule_state.dtype == torch.float32
+        d = GatedOuterSpec()
+        d.w_in, d.w_out, d.f_bias, d.lower, d.gain = self._held(m.w_in, m.w_out, m.f_bias, m.lower, m.gain)
+        d.rule_state, d.slot_stride = rule_state.data_ptr(), int(rule_state.stride(0))
+        self.keep.append(rule_state)
+        d.heads, d.dim, d.vdim, d.eps = m.heads, m.dim, m.vdim, m.norm_eps
+        return self._made(L.library().gibbs_plan_body_gated_outer(self.handle, ctypes.byref(d)))
+
+    def differential_attention(self, m, *, kpages: torch.Tensor, vpages: torch.Tensor, group: int, stored) -> int:
+        """The differential-attention mixer `m` (parts/diff_attention.py) over its pages [num_pages, kv_heads, page_size, size]."""
+        from ..ops import ROPE_VARIANTS
+        assert kpages.is_contiguous() and vpages.is_contiguous() and kpages.shape[:-1] == vpages.shape[:-1]
+        d = DiffAttentionSpec()
+        d.w_in, d.w_out, d.q_gain, d.k_gain, d.lam = self._held(m.w_in, m.w_out, m.q_gain, m.k_gain, m.lam)
+        d.rot = d.variant = d.table_len = 0
+        if m.rot is not None:
+            d.inv_freq, d.cos_sin = self._held(m.rot.inv_freq, m.rot.cos_sin)
+            d.rot, d.variant = int(m.rot.rotary_dim), ROPE_VARIANTS[m.rot.variant]
+            d.table_len = 0 if m.rot.cos_sin is None else int(m.rot.cos_sin.shape[0])
+        d.kpages, d.vpages = kpages.data_ptr(), vpages.data_ptr()
+        self.keep += [kpages, vpages]
+        d.in_rows, d.heads, d.kv_heads, d.dim, d.vdim = m.w_in.shape[0], m.heads, m.kv_heads, m.head_dim, m.v_head_dim
+        d.k_stored, d.v_stored = stored
+        d.window, d.chunk, d.gate_off = int(m.window or 0), m.chunk, m.gate_off
+        d.num_pages, d.page_size, d.group = int(kpages.shape[0]), int(kpages.shape[2]), int(group)
+        d.scale, d.eps, d.out_scale = m.scale, m.norm_eps, 1.0 - m.diff
+        return self._made(L.library().gibbs_plan_body_diff_attention(self.handle, ctypes.byref(d)))
+
     def logit_softcap(self, cap: float) -> None:
         self._made(L.library().gibbs_plan_logit_softcap(self.handle, float(cap)))
 
@@ -335,15 +405,17 @@ class NativePlan:
 
     def moe(self, m) -> int:
         """The mixture-of-experts feed-forward `m` (parts/moe.py)."""
-        from ..ops import ACTIVATIONS
+        from ..ops import ACTIVATIONS, MOE_SCORES
         d = MoeSpec()
         d.router, d.router_bias, d.gate, d.up, d.down = self._held(m.router, m.router_bias, m.w_gate, m.w_up, m.w_down)
         d.shared_gate_up, d.shared_down, d.shared_gate = self._held(m.shared_gate_up, m.shared_down, m.shared_gate)
         d.experts, d.top, d.F, d.act = m.experts, m.top, m.inter, ACTIVATIONS[m.activation]
         d.shared_F, d.shared_act = m.shared_inter, ACTIVATIONS[m.shared_activation]
         body = self._made(L.library().gibbs_plan_body_moe(self.handle, ctypes.byref(d)))
-        if m.scores == "softmax_all" or m.identity:
-            self._made(L.library().gibbs_plan_moe_scores(self.handle, body, int(m.scores == "softmax_all"), int(m.identity)))
+        if m.scores != "softmax_top" or m.identity:
+            self._made(L.library().gibbs_plan_moe_scores(self.handle, body, MOE_SCORES[m.scores], int(m.identity)))
+        if m.weigh == "input":
+            self._made(L.library().gibbs_plan_moe_weigh_input(self.handle, body))
         return body
 
     def glu_clamped(self, body: int, *, alpha: float, limit: float) -> None:
@@ -502,6 +574,10 @@ class NativePlan:
         plan = cls(rt, model.spec.hidden, model.spec.vocab, model.table, model.head, model.head_packed)
         if model.spec.embedding_scale != 1.0 or model.embedding_inv_freq is not None:
             plan.embedding(model.spec.embedding_scale, model.embedding_inv_freq)
+        if model.embedding_norm is not None:
+            if model.spec.embedding_norm.kind != "rms":
+                raise ValueError(f"a norm of kind {model.spec.embedding_norm.kind!r} on the embedding is not implemented ('rms')")
+            plan.embedding_norm(model.embedding_norm.gain, model.embedding_norm.spec.eps)
         if model.spec.streams != 1:
             plan.streams(model.spec.streams)
         tables = model.spec.embedding_tables

@@ -19,11 +19,14 @@ from .base import Norm, Runtime, register_norm
 @register_norm("rms")
 class RMSNorm(Norm):
     def tensor_decls(self) -> List[TensorDecl]:
-        return [TensorDecl(self.spec.weight, (self.width,), FLOAT32, init="gain")]
+        names = [self.spec.weight] + ([self.spec.scale] if self.spec.scale is not None else [])
+        return [TensorDecl(n, (self.width,), FLOAT32, init="gain") for n in names]
 
     def bind(self, weights: WeightStore, rt: Runtime) -> None:
         self.rt = rt
         self.gain = weights[self.spec.weight]
+        if self.spec.scale is not None:      # (a scale per channel on the normed row: one more factor of the gain)
+            self.gain = (self.gain * weights[self.spec.scale]).contiguous()
 
     def fold_gain(self) -> torch.Tensor:
         """Hands the gain over to whoever multiplies it into the matrices that read the normed

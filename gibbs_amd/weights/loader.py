@@ -30,7 +30,7 @@ class TensorDecl:
     name: str
     shape: Tuple[int, ...]
     dtype: str = COMPUTE                    # COMPUTE | FLOAT32 | INT32
-    init: str = "normal"                    # random-weights mode: normal | gain | bias | zeros
+    init: str = "normal"                    # random-weights mode: normal | gain | bias | zeros | unit (uniform in [0, 1))
     alt_shapes: Tuple[Tuple[int, ...], ...] = ()   # other stored shapes of the same data
 
     def resolved_dtype(self, compute_dtype: torch.dtype) -> torch.dtype:

@@ -40,6 +40,8 @@ def random_tensor(decl: TensorDecl, seed: int, store_dtype: torch.dtype, std: fl
         t = torch.randn(decl.shape, generator=g, dtype=torch.float32) * bias_std
     elif decl.init == "zeros":
         t = torch.zeros(decl.shape, dtype=torch.float32)
+    elif decl.init == "unit":
+        t = torch.rand(decl.shape, generator=g, dtype=torch.float32)
     else:
         t = torch.randn(decl.shape, generator=g, dtype=torch.float32) * std
     keep32 = decl.dtype == FLOAT32 or len(decl.shape) <= 1
@@ -79,6 +81,8 @@ def random_weights_on_device(decls: Iterable[TensorDecl], seed: int, compute_dty
             out[d.name] = t.to(want)
         elif d.init == "zeros":
             out[d.name] = torch.zeros(d.shape, dtype=want, device=device)
+        elif d.init == "unit":
+            out[d.name] = torch.rand(d.shape, generator=g, dtype=torch.float32, device=device).to(want)
         else:
             scale = bias_std if d.init == "bias" else std
             out[d.name] = (torch.randn(d.shape, generator=g, dtype=torch.float32, device=device) * scale).to(want)
