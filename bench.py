@@ -361,9 +361,34 @@ def litizen_shape(width: int, ff: int, layers: int, vocab: int) -> dict:
             "layers": [dict(kinds[i % 3], mlp=mlps[i % 2]) for i in range(layers)]}
 
 
+def gumozen_shape(width: int, ff: int, layers: int, vocab: int) -> dict:
+    """A Gumozen model of `layers` layers (gated outer-product recurrence, differential attention, latent attention in turn) whose
+    sizes resemble a real model's at this width: recurrent heads of 128 x 128; two maps of 64 over values of 128 in groups of four,
+    half of every map rotated with scaled frequencies, chunks of 1,024; latent heads of 64 over a cached latent of 128, queries
+    through a latent of half the width, every latent layer behind the first reading the first one's latent; 16 experts of a
+    quarter of the dense width, of which a token takes 4."""
+    heads = max(1, width // 128)
+    kinds = [
+        {"type": "hgrn2", "mixer": {"heads": heads, "dim": 128, "vdim": 128}},
+        {"type": "attention", "mixer": {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 64, "vdim": 128, "scale": 0.125, "diff": 0.5,
+                                        "mask": {"size": 1024},
+                                        "rot": {"base": 500000.0, "dims": 32, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}},
+        {"type": "latent_attention", "mixer": {"heads": width // 64, "dim": 64, "vdim": 64, "kv_rank": 128, "q_rank": width // 2, "scale": 0.125}},
+    ]
+    mlp = {"kind": "moe", "expert": {"ff": ff // 4}, "router": {"experts": 16, "top": 4}}
+    made = []
+    for i in range(layers):
+        layer = dict(kinds[i % 3], mlp=mlp)
+        if i % 3 == 2 and i > 2:
+            layer["mixer"] = dict(layer["mixer"], kv_from=2)
+        made.append(layer)
+    return {"architecture": "Gumozen", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": made}
+
+
 # design -> (its name, its shape, the closest model the framework had, that model's shape at equal sizes)
 BESIDE = {"zokepel": ("Zokepel", zokepel_shape, "LFM2", lfm2_shape), "rukosun": ("Rukosun", rukosun_shape, "LFM2", lfm2_attention_shape),
-          "ruzinex": ("Ruzinex", ruzinex_shape, "LFM2", lfm2_attention_shape), "litizen": ("Litizen", litizen_shape, "Ruzinex", ruzinex_shape)}
+          "ruzinex": ("Ruzinex", ruzinex_shape, "LFM2", lfm2_attention_shape), "litizen": ("Litizen", litizen_shape, "Ruzinex", ruzinex_shape),
+          "gumozen": ("Gumozen", gumozen_shape, "Litizen", litizen_shape)}
 
 
 def engine_of(shape: dict, dtype: str, max_requests: int, context: int):
@@ -381,7 +406,7 @@ def engine_of(shape: dict, dtype: str, max_requests: int, context: int):
 
 
 def compare_designs(args) -> int:
-    """`--design zokepel` / `rukosun` / `ruzinex` / `litizen`: prefill and decode speed of that design at a few sizes beside LFM2 (Litizen: beside Ruzinex) at equal
+    """`--design NAME`: prefill and decode speed of that design at a few sizes beside the closest one in `BESIDE` at equal
     width, depth, feed-forward and vocabulary (random weights), with the kernels that each one's time goes to.  One
     JSON line."""
     import faulthandler
@@ -443,10 +468,10 @@ def compare_designs(args) -> int:
 
 def main() -> int:
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", choices=["lfm2", "zokepel", "rukosun", "ruzinex", "litizen"], default="lfm2",
+    ap.add_argument("--design", choices=["lfm2"] + sorted(BESIDE), default="lfm2",
                     help="zokepel, rukosun, ruzinex: that design beside LFM2 at equal sizes instead of the headline workload; "
-                         "litizen: beside Ruzinex, the closest design the framework had")
-    ap.add_argument("--sizes", choices=["small", "medium", "all"], default="medium", help="sizes of --design zokepel / rukosun / ruzinex / litizen")
+                         "litizen: beside Ruzinex, gumozen: beside Litizen, the closest designs the framework had")
+    ap.add_argument("--sizes", choices=["small", "medium", "all"], default="medium", help="sizes of --design (any but lfm2)")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=128)
     ap.add_argument("--warmup", type=int, default=16)

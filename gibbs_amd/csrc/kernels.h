@@ -110,6 +110,11 @@ int gibbs_diff_finish(const void* att, int vs, const void* gate, long ld_gate, c
 int gibbs_gated_outer_prep(const void* raw, long ld, int dtype, const float* bias, const float* lower, float* q, float* f, float* k,
                            float* v, int n_rows, int H, int D, int V, hipStream_t stream);
 int gibbs_gated_outer_step_takes(int D, int V);
+int gibbs_gated_outer_chunks_take(int D, int V);
+long gibbs_gated_outer_chunks_workspace(int rows, int n_req, int H, int D, int V);
+int gibbs_gated_outer_chunks(const void* raw, long ld, int dtype, const float* bias, const float* lower, const float* gain, float eps,
+                             float* state, long slot_stride, const int* cu, const int* slot, void* out, float* workspace, int n_rows,
+                             int n_req, int H, int D, int V, hipStream_t stream);
 int gibbs_gated_outer_step(const void* raw, long ld, int dtype, const float* bias, const float* lower, const float* gain, float eps,
                            float* state, long slot_stride, const int* slot, void* out, int n_req, int H, int D, int V, hipStream_t stream);
 int gibbs_gated_outer_rule(const float* q, const float* k, const float* v, const float* decay, float* state, long slot_stride,

@@ -48,6 +48,7 @@ constexpr int SKINNY_ROWS = 64;           // rows up to which a plain product ta
 constexpr int SKINNY_ROWS_F32_OUT = 48;   // the same for float32 output (the head: it streams faster than the tiled product)
 constexpr int ACT_CLAMPED = 4;            // the gated feed-forward's clamped activation (activation.h: ACT_CLAMPED_SWISH)
 constexpr int SSD_CHUNKED_ROWS = 256;     // rows of one request from which the state-space rule runs in chunks
+constexpr int GATED_CHUNKED_ROWS = 96;    // rows of a request from which the gated outer-product rule runs in chunks
 constexpr int MATRIX_SLICE_PAGES = 510;   // page ids of a key slice that the decode attention's matrix-core walk keeps in LDS
 
 // Ranges of k that the few-row product is cut into so that at least `want_blocks` workgroups run (a
@@ -1130,8 +1131,8 @@ struct DiffAttnBody : Body {
 
 // ---- gated outer-product recurrence
 // One product gives [a | z | v] of the rows; per head q = silu(a), f = l + (1 - l) sigmoid(z + b), S = diag(f) S + (1 - f) v',
-// read-out S' q normed per head, times a gain, projected back.  A step of one token per request is one kernel between the two
-// products; other steps prepare their rows and walk (gated_outer.hip, recurrent.hip).
+// read-out S' q normed per head, times a gain, projected back.  Decoded tokens are one kernel between the two products, long
+// portions three (the rule in chunks), short ones prepare their rows and walk (gated_outer.hip, recurrent.hip).
 struct GatedOuterBody : Body {
   Matrix in, out;
   int H = 0, D = 0, V = 0;
@@ -1147,21 +1148,31 @@ struct GatedOuterBody : Body {
     const long C = (long)H * D, HV = (long)H * V;
     void* raw = e.linear(h, in, N, false, false, false, nullptr);
     void* y = e.take((long)N * HV * e.esize);
-    if (e.rows_are_requests() && gibbs_gated_outer_step_takes(D, V)) {
-      RUN(e, gibbs_gated_outer_step(raw, in.O, e.p.dtype, bias, lower, gain, eps, rule_state, slot_stride, a.slot, y, a.n_req, H, D, V, a.stream));
-    } else {
-      float* q = (float*)e.take((long)N * C * 4);
-      float* f = (float*)e.take((long)N * C * 4);
-      float* k = (float*)e.take((long)N * C * 4);
-      float* v = (float*)e.take((long)N * HV * 4);
-      RUN(e, gibbs_gated_outer_prep(raw, in.O, e.p.dtype, bias, lower, q, f, k, v, N, H, D, V, a.stream));
-      float* o = (float*)e.take((long)N * HV * 4);
-      RUN(e, gibbs_gated_outer_rule(q, k, v, f, rule_state, slot_stride, a.cu, a.slot, o, a.n_req, H, D, V, a.stream));
+    // requests at the head of the batch that bring one row each (row n is request n's) take the step kernel; the others the
+    // rule in chunks where one of them brings a long portion, else the walk
+    const int lead = !gibbs_gated_outer_step_takes(D, V) ? 0 : (e.rows_are_requests() ? N : a.lead_single);
+    const int rest = N - lead, reqs = a.n_req - lead;
+    if (lead > 0) RUN(e, gibbs_gated_outer_step(raw, in.O, e.p.dtype, bias, lower, gain, eps, rule_state, slot_stride, a.slot, y, lead, H, D, V, a.stream));
+    if (rest > 0 && a.max_q >= GATED_CHUNKED_ROWS && gibbs_gated_outer_chunks_take(D, V)) {
+      float* work = (float*)e.take(gibbs_gated_outer_chunks_workspace(rest, reqs, H, D, V) * 4);
+      RUN(e, gibbs_gated_outer_chunks(raw, in.O, e.p.dtype, bias, lower, gain, eps, rule_state, slot_stride, a.cu + lead, a.slot + lead, y, work, rest, reqs,
+                                      H, D, V, a.stream));
+      e.give(work);
+    } else if (rest > 0) {
+      float* q = (float*)e.take(rest * C * 4);
+      float* f = (float*)e.take(rest * C * 4);
+      float* k = (float*)e.take(rest * C * 4);
+      float* v = (float*)e.take(rest * HV * 4);
+      float* o = (float*)e.take(rest * HV * 4);
+      RUN(e, gibbs_gated_outer_prep((char*)raw + (long)lead * in.O * e.esize, in.O, e.p.dtype, bias, lower, q, f, k, v, rest, H, D, V, a.stream));
+      // (the walk's rows are counted from the step's first: its operands start `lead` rows earlier, and are not read there)
+      RUN(e, gibbs_gated_outer_rule(q - lead * C, k - lead * C, v - lead * HV, f - lead * C, rule_state, slot_stride, a.cu + lead, a.slot + lead,
+                                    o - lead * HV, reqs, H, D, V, a.stream));
       e.give(q);
       e.give(f);
       e.give(k);
       e.give(v);
-      RUN(e, gibbs_head_norm_gate(o, gain, V, nullptr, 0, y, e.p.dtype, N, H, V, eps, 0, a.stream));
+      RUN(e, gibbs_head_norm_gate(o, gain, V, nullptr, 0, (char*)y + lead * HV * e.esize, e.p.dtype, rest, H, V, eps, 0, a.stream));
       e.give(o);
     }
     e.give(raw);

@@ -98,6 +98,9 @@ _SIGNATURES = {
                                c_void_p],
     "gibbs_gated_outer_step": [c_void_p, c_long, c_int, c_void_p, c_void_p, c_void_p, c_float, c_void_p, c_long, c_void_p, c_void_p, c_int, c_int,
                                c_int, c_int, c_void_p],
+    "gibbs_gated_outer_chunks": [c_void_p, c_long, c_int, c_void_p, c_void_p, c_void_p, c_float, c_void_p, c_long, c_void_p, c_void_p, c_void_p,
+                                 c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
+    "gibbs_head_norm_gate": [c_void_p, c_void_p, c_int, c_void_p, c_long, c_void_p, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p],
     "gibbs_gated_outer_rule": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
                                c_void_p],
     "gibbs_moe_gemm_weighted": [c_void_p, c_long, c_int, c_void_p, c_void_p, c_long, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_int,
@@ -178,6 +181,9 @@ _VALUE_SIGNATURES = {
     "gibbs_rule_fused_rows": ([], c_int),
     "gibbs_linear_splits": ([c_int, c_int, c_int, c_int, c_long, c_void_p, c_void_p, c_int, c_int, c_int], c_int),
     "gibbs_skinny_residual_workspace": ([c_int, c_int, c_int], c_long),
+    "gibbs_gated_outer_chunks_take": ([c_int, c_int], c_int),
+    "gibbs_gated_outer_step_takes": ([c_int, c_int], c_int),
+    "gibbs_gated_outer_chunks_workspace": ([c_int, c_int, c_int, c_int, c_int], c_long),
     "gibbs_ssd_chunked_workspace": ([c_int, c_int, c_int, c_int], c_long),
 }
 
