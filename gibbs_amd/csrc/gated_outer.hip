@@ -132,10 +132,15 @@ __global__ __launch_bounds__(STEP_THREADS) void gated_outer_step_kernel(const T*
 // operands.  Every exponent is a sum over few segments, and the two factors that a score's decay is split into never grow:
 //   s in an earlier segment than t   e^(b_t) and e^(B_J - b_s + segments between)
 //   s in the first half of t's segment, t in the second   both about the border between the halves
-//   both in the same half (8 tokens)   about the half's middle: a factor may grow over at most four tokens, and log f is kept
-//   above -19.4 here (f at least 3.7e-9: what is left of the state then is below the rounding of what is added), e^78
-// so nothing overflows that is used.  The order of additions differs from the walk's: results agree to rounding.
+//   both in the same half (8 tokens)   about the half's middle: a factor may grow over at most four tokens, and log2 f is kept
+//   above -28 here (f at least 3.7e-9: what is left of the state then is below the rounding of what is added), 2^112
+// so nothing overflows that is used.  Logarithms are to base 2: the vector unit's own exponential, logarithm and reciprocal
+// (one unit in the last place) are what the many factors cost.  The order of additions differs from the walk's: results
+// agree to rounding.
 constexpr int CHUNK = 64, SEG = 16, CT = 512, CWAVES = CT / WAVE, MAX_VT = 2;
+constexpr float LOG2E = 1.44269504088896340736f;
+__device__ __forceinline__ float exp2_of(float x) { return __builtin_amdgcn_exp2f(x); }
+__device__ __forceinline__ float rcp_of(float x) { return __builtin_amdgcn_rcpf(x); }
 typedef __attribute__((__vector_size__(4 * sizeof(float)))) float floatx4;
 struct ChunkedArgs {
   const void* raw;            // [rows, ld]: [a | z | v]
@@ -148,6 +153,8 @@ struct ChunkedArgs {
   const int* cu; const int* slot;
   void* out;                  // [rows, H * V]
   int n_req, H, D, V;
+  int d_shift, v_shift;       // log2 of the next powers of two of D's multiple of 16 and of V / 8
+  int v8;                     // values are loaded 8 at a time
 };
 // the request and the chunk of it that place `p` stands for (false: none)
 __device__ __forceinline__ bool chunk_of(const ChunkedArgs& a, int p, int* t0, int* rows) {
@@ -164,41 +171,63 @@ __device__ __forceinline__ bool chunk_of(const ChunkedArgs& a, int p, int* t0, i
 }
 // q (optional), k and b of the chunk's tokens into LDS rows of `lq` floats (channels from D to Dp and tokens beyond the end:
 // q = k = 0, no decay), and the segments' sums tot [4][lq].
-template <typename T>
+template <typename T, bool Q>
 __device__ __forceinline__ void chunk_gates(const ChunkedArgs& a, int h, int t0, int rows, int Dp, int lq, float* sq, float* sk, float* sb, float* tot) {
-  const int C = a.H * a.D;
-  for (int idx = threadIdx.x; idx < (CHUNK / SEG) * Dp; idx += CT) {
-    const int seg = idx / Dp, i = idx % Dp;
+  const int C = a.H * a.D, span = 1 << a.d_shift;
+  for (int idx = threadIdx.x; idx < (CHUNK / SEG) * span; idx += CT) {
+    const int seg = idx >> a.d_shift, i = idx & (span - 1);
+    if (i >= Dp) continue;
     const bool live = i < a.D;
     const int c = h * a.D + (live ? i : 0);
-    const T* at = (const T*)a.raw + (size_t)(t0 + seg * SEG) * a.ld + c;
-    const int here = min(SEG, rows - seg * SEG);
-    float z[SEG], q[SEG];
+    const T* at = (const T*)a.raw + (size_t)t0 * a.ld + c;
+    T z[SEG], q[SEG];
 #pragma unroll
-    for (int t = 0; t < SEG; ++t) {
-      const bool in = live && t < here;
-      z[t] = in ? to_float(at[(size_t)t * a.ld + C]) : 0.f;
-      q[t] = (in && sq) ? to_float(at[(size_t)t * a.ld]) : 0.f;
+    for (int t = 0; t < SEG; ++t) {      // (rows beyond the end: the last one again, masked below)
+      const T* row = at + (size_t)min(seg * SEG + t, rows - 1) * a.ld;
+      z[t] = row[C];
+      if constexpr (Q) q[t] = row[0];
     }
     const float bias = a.bias[c], l = a.lower[c];
     float run = 0.f;
 #pragma unroll
     for (int t = 0; t < SEG; ++t) {
       const int row = seg * SEG + t;
-      const Gate g = gate_of(z[t] + bias, l);
-      const bool in = live && t < here;
-      if (in) run += g.k < 0.5f ? log1pf(-g.k) : logf(fmaxf(g.f, 3.7e-9f));
-      sk[row * lq + i] = in ? g.k : 0.f;
+      const bool in = live && row < rows;
+      const float x = to_float(z[t]) + bias;
+      const float e = exp2_of(-fabsf(x) * LOG2E), inv = rcp_of(1.0f + e), ei = e * inv;
+      const float f = fmaf(1.0f - l, x >= 0.f ? inv : ei, l), k = (1.0f - l) * (x >= 0.f ? ei : inv);
+      run += in ? __builtin_amdgcn_logf(fmaxf(f, 3.7252903e-9f)) : 0.f;
+      sk[row * lq + i] = in ? k : 0.f;
       sb[row * lq + i] = run;
-      if (sq) sq[row * lq + i] = q[t] * sigm(q[t]);
+      if constexpr (Q) {
+        const float y = to_float(q[t]);
+        sq[row * lq + i] = in ? y * rcp_of(1.0f + exp2_of(-y * LOG2E)) : 0.f;
+      }
     }
     tot[seg * lq + i] = run;
   }
 }
+__device__ __forceinline__ void load_eight(const bf16* p, float* f) { unpack8(*(const uint4*)p, f); }
+__device__ __forceinline__ void load_eight(const float* p, float* f) {
+  const float4 a = *(const float4*)p, b = *(const float4*)(p + 4);
+  f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w; f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w;
+}
 template <typename T>
 __device__ __forceinline__ void chunk_values(const ChunkedArgs& a, int h, int t0, int rows, int Vp, int lv, float* sv) {
   const T* at = (const T*)a.raw + (size_t)t0 * a.ld + 2 * a.H * a.D + h * a.V;
-#pragma unroll 4
+  if (a.v8) {
+    const int span = 1 << a.v_shift;
+#pragma unroll 2
+    for (int idx = threadIdx.x; idx < CHUNK * span; idx += CT) {
+      const int t = idx >> a.v_shift, j = (idx & (span - 1)) * 8;
+      if (j >= Vp) continue;
+      float f[8] = {};
+      if (t < rows && j < a.V) load_eight(at + (size_t)t * a.ld + j, f);
+      *(float4*)(sv + t * lv + j) = make_float4(f[0], f[1], f[2], f[3]);
+      *(float4*)(sv + t * lv + j + 4) = make_float4(f[4], f[5], f[6], f[7]);
+    }
+    return;
+  }
   for (int idx = threadIdx.x; idx < CHUNK * Vp; idx += CT) {
     const int t = idx / Vp, j = idx % Vp;
     sv[t * lv + j] = (t < rows && j < a.V) ? to_float(at[(size_t)t * a.ld + j]) : 0.f;
@@ -216,19 +245,21 @@ __global__ __launch_bounds__(CT) void gated_outer_chunk_state_kernel(ChunkedArgs
   int t0, rows;
   if (!chunk_of(a, blockIdx.x, &t0, &rows)) return;
   const int h = blockIdx.y;
-  chunk_gates<T>(a, h, t0, rows, Dp, lq, nullptr, sk, sb, tot);
+  chunk_gates<T, false>(a, h, t0, rows, Dp, lq, nullptr, sk, sb, tot);
   chunk_values<T>(a, h, t0, rows, Vp, lv, sv);
   __syncthreads();
   // k_s times the decay from behind s to the chunk's end
-  for (int idx = threadIdx.x; idx < CHUNK * Dp; idx += CT) {
-    const int t = idx / Dp, i = idx % Dp, seg = t / SEG;
-    float e = tot[seg * lq + i] - sb[t * lq + i];
-    for (int m = seg + 1; m < CHUNK / SEG; ++m) e += tot[m * lq + i];
-    sk[t * lq + i] *= expf(e);
+  for (int idx = threadIdx.x; idx < (CHUNK / SEG) << a.d_shift; idx += CT) {
+    const int seg = idx >> a.d_shift, i = idx & ((1 << a.d_shift) - 1);
+    if (i >= Dp) continue;
+    float rest = tot[seg * lq + i];
+    for (int m = seg + 1; m < CHUNK / SEG; ++m) rest += tot[m * lq + i];
+#pragma unroll
+    for (int t = seg * SEG; t < seg * SEG + SEG; ++t) sk[t * lq + i] *= exp2_of(rest - sb[t * lq + i]);
   }
   if (threadIdx.x < a.D) {
     const int i = threadIdx.x;
-    a.decay[((size_t)blockIdx.x * a.H + h) * a.D + i] = expf(tot[i] + tot[lq + i] + tot[2 * lq + i] + tot[3 * lq + i]);
+    a.decay[((size_t)blockIdx.x * a.H + h) * a.D + i] = exp2_of(tot[i] + tot[lq + i] + tot[2 * lq + i] + tot[3 * lq + i]);
   }
   __syncthreads();
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE, lr = lane % 16, g = lane / 16;
@@ -309,7 +340,7 @@ __global__ __launch_bounds__(CT) void gated_outer_chunk_out_kernel(ChunkedArgs a
   int t0, rows;
   if (!chunk_of(a, blockIdx.x, &t0, &rows)) return;
   const int h = blockIdx.y;
-  chunk_gates<T>(a, h, t0, rows, Dp, lq, sq, sk, sb, tot);
+  chunk_gates<T, true>(a, h, t0, rows, Dp, lq, sq, sk, sb, tot);
   chunk_values<T>(a, h, t0, rows, Vp, lv, sv);
   __syncthreads();
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE, lr = lane % 16, g = lane / 16;
@@ -342,7 +373,7 @@ __global__ __launch_bounds__(CT) void gated_outer_chunk_out_kernel(ChunkedArgs a
       const float qv[4] = {q4.x, q4.y, q4.z, q4.w}, kv[4] = {k4.x, k4.y, k4.z, k4.w};
       const float ek[4] = {r4.x - y4.x, r4.y - y4.y, r4.z - y4.z, r4.w - y4.w};
 #pragma unroll
-      for (int j = 0; j < 4; ++j) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(qv[j] * expf(eq[j]), kv[j] * expf(ek[j]), acc, 0, 0, 0);
+      for (int j = 0; j < 4; ++j) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(qv[j] * exp2_of(eq[j]), kv[j] * exp2_of(ek[j]), acc, 0, 0, 0);
     }
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
@@ -355,11 +386,13 @@ __global__ __launch_bounds__(CT) void gated_outer_chunk_out_kernel(ChunkedArgs a
   }
   __syncthreads();
   // q_t times the decay from the chunk's start to t
-  for (int idx = threadIdx.x; idx < CHUNK * Dp; idx += CT) {
-    const int t = idx / Dp, i = idx % Dp, seg = t / SEG;
-    float e = sb[t * lq + i];
-    for (int m = 0; m < seg; ++m) e += tot[m * lq + i];
-    sq[t * lq + i] *= expf(e);
+  for (int idx = threadIdx.x; idx < (CHUNK / SEG) << a.d_shift; idx += CT) {
+    const int seg = idx >> a.d_shift, i = idx & ((1 << a.d_shift) - 1);
+    if (i >= Dp) continue;
+    float before = 0.f;
+    for (int m = 0; m < seg; ++m) before += tot[m * lq + i];
+#pragma unroll
+    for (int t = seg * SEG; t < seg * SEG + SEG; ++t) sq[t * lq + i] *= exp2_of(before + sb[t * lq + i]);
   }
   __syncthreads();
   const float* s0 = a.u + ((size_t)blockIdx.x * a.H + h) * a.D * a.V;
@@ -410,22 +443,27 @@ __global__ __launch_bounds__(CT) void gated_outer_chunk_out_kernel(ChunkedArgs a
       if (lr == 0) red[wave * CHUNK + I * SEG + g * 4 + i] = ss;
     }
   __syncthreads();
+  if (threadIdx.x < CHUNK) {
+    float total = 0.f;
 #pragma unroll
-  for (int I = 0; I < CHUNK / SEG; ++I)
+    for (int w = 0; w < CWAVES; ++w) total += red[w * CHUNK + threadIdx.x];
+    red[threadIdx.x] = 1.0f / sqrtf(total / (float)a.V + a.eps);
+  }
+  __syncthreads();
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int t = I * SEG + g * 4 + i;
-      if (t >= rows) continue;
-      float total = 0.f;
+  for (int v = 0; v < MAX_VT; ++v) {
+    const int col = (wave + v * CWAVES) * 16 + lr;
+    if (col >= a.V) break;
+    const float gain = a.gain[col];
+    T* out = (T*)a.out + ((size_t)t0 * a.H + h) * a.V + col;
 #pragma unroll
-      for (int w = 0; w < CWAVES; ++w) total += red[w * CHUNK + t];
-      const float inv = 1.0f / sqrtf(total / (float)a.V + a.eps);
+    for (int I = 0; I < CHUNK / SEG; ++I)
 #pragma unroll
-      for (int v = 0; v < MAX_VT; ++v) {
-        const int col = (wave + v * CWAVES) * 16 + lr;
-        if (col < a.V) ((T*)a.out)[((size_t)(t0 + t) * a.H + h) * a.V + col] = from_float<T>(acc[v][I][i] * inv * a.gain[col]);
+      for (int i = 0; i < 4; ++i) {
+        const int t = I * SEG + g * 4 + i;
+        if (t < rows) out[(size_t)t * a.H * a.V] = from_float<T>(acc[v][I][i] * red[t] * gain);
       }
-    }
+  }
 }
 size_t chunk_state_lds(int D, int V) {
   const int lq = (D + 15) / 16 * 16 + 4, lv = (V + 15) / 16 * 16 + 4;
@@ -471,7 +509,11 @@ GIBBS_EXPORT int gibbs_gated_outer_chunks(const void* raw, long ld, int dtype, c
   GIBBS_REQUIRE(H > 0 && H <= 65535 && gibbs_gated_outer_chunks_take(D, V) && ld >= (long)H * (2 * D + V) && slot_stride >= (long)H * D * V,
                 "gated_outer_chunks: heads=%d D=%d V=%d", H, D, V);
   const int places = ceil_div(n_rows, CHUNK) + n_req;      // (more than the requests' chunks can be)
-  ChunkedArgs a{raw, ld, bias, lower, gain, eps, workspace, workspace + (size_t)places * H * D * V, state, slot_stride, cu, slot, out, n_req, H, D, V};
+  ChunkedArgs a{raw, ld, bias, lower, gain, eps, workspace, workspace + (size_t)places * H * D * V, state, slot_stride, cu, slot, out, n_req, H, D, V, 4, 0, 0};
+  while ((1 << a.d_shift) < D) ++a.d_shift;
+  while ((1 << a.v_shift) * 8 < V) ++a.v_shift;
+  if (V % 16) a.v_shift = std::max(a.v_shift, 1);      // (the zeros up to the next multiple of 16 are written as well)
+  a.v8 = V % 8 == 0 && ld % 8 == 0 && (2L * H * D) % 8 == 0 && ((uintptr_t)raw % 16) == 0;
   if (dtype == GIBBS_F32) { if (launch_chunks<float>(a, places, stream)) return 1; }
   else if (dtype == GIBBS_BF16) { if (launch_chunks<bf16>(a, places, stream)) return 1; }
   else return gibbs_fail("gated_outer_chunks: unknown dtype %d", dtype);
