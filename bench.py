@@ -95,7 +95,7 @@ def time_prefill(engine, runs: int = 5, n_tokens: int = PROMPT_LEN, warmups: int
 
 
 def time_decode(engine, batch: int, steps: int, warmup: int, runs: int = RUNS, profile: bool = False,
-                prompt_len: int = PROMPT_LEN, most: int = 8):
+                prompt_len: int = PROMPT_LEN, most: int = 8, use_graph: bool = True):
     """Median seconds for exactly `steps` decode steps of `batch` requests that each hold a
     `prompt_len`-token prompt (greedy sampling on the device), the requests' lengths at the middle of that
     run, and, with `profile`, the kernels of one more run by their share of its device time."""
@@ -108,7 +108,7 @@ def time_decode(engine, batch: int, steps: int, warmup: int, runs: int = RUNS, p
     for i, rid in enumerate(rids):
         logits = engine.step([(rid, seeded_prompt(i, prompt_len, vocab), [prompt_len - 1])])
         first.append(int(logits.argmax(-1).item()))
-    loop = DecodeLoop(engine, rids, first)
+    loop = DecodeLoop(engine, rids, first, use_graph=use_graph)
     if warmup > 0:
         loop.run(warmup)
     samples = []
@@ -417,8 +417,8 @@ def compare_designs(args) -> int:
     from gibbs_amd import roofline as R
     faulthandler.enable()       # (a crash inside a library names the Python frame it came from)
     # The kernels' shares come from the profiler, which sometimes dies when it stops after replays of captured
-    # graphs; they are therefore measured by a child process of their own, first, and a child that fails costs
-    # the listing only.  This process then measures the times with no profiler loaded.
+    # graphs; they are therefore measured by a child process of their own, first, over steps without graphs (the
+    # same kernels), and a child that fails costs the listing only.  This process then measures the times with no profiler loaded.
     listed = {}
     if not args.no_kernels and not args.kernels_child:
         import subprocess
@@ -449,7 +449,7 @@ def compare_designs(args) -> int:
                 ids = seeded_prompt(5, args.prefill_tokens, vocab)
                 row["prefill_kernels"] = kernel_shares(lambda: (engine.step([("k", ids, [len(ids) - 1])]), engine.release("k")), most=14)
             print(f"[bench] {design} width {width}: decode", file=sys.stderr, flush=True)
-            dt, seq_lens, top = time_decode(engine, args.batch, args.steps, args.warmup, profile=profile, prompt_len=args.prompt_len, most=14)
+            dt, seq_lens, top = time_decode(engine, args.batch, args.steps, args.warmup, profile=profile, prompt_len=args.prompt_len, most=14, use_graph=not profile)
             row["decode_tok_s"] = round(args.batch * args.steps / dt, 1)
             row["decode_ms_per_step"] = round(dt / args.steps * 1e3, 4)
             row["decode_frac_of_hbm"] = round(R.decode_bytes(engine, seq_lens) / (dt / args.steps) / R.HBM_BYTES_PER_S, 4)
