@@ -9,7 +9,7 @@ into it.
               `mask.size` positions counted from 0; q and k normed per head and map, then the first `rot.dims` channels turned
               (pairs (i, i + dims/2), frequencies with the smooth three-band scaling of `rot.scaling`); o = a_1 - lambda a_2,
               divided by its root mean square, times 1 - `diff`, times one sigmoid gate per head
-  hgrn2       linear attention whose forget gate f = l + (1 - l) sigmoid(W_f h + b) also decides what is written:
+  hgrn2       a recurrence per head with a decay per channel, f = l + (1 - l) sigmoid(W_f h + b), and its complement as the key:
               S = diag(f) S + (1 - f) v', read-out S' q normed per head
   latent_attention  queries through a normed latent, keys and values of all heads from a small normed latent that is cached;
               no positions; a layer with `kv_from` reads an earlier layer's cached latent with its own up-projections

@@ -1,4 +1,4 @@
-"""Gated outer-product mixer (HGRN2): linear attention in which the forget gate also decides what is written.
+"""Gated outer-product mixer (HGRN2): a decayed state per head in which the complement of the decay stands for the key.
 
 With h the mixer's input, per head, q = silu(W_q h) [dim], v = W_v h [vdim] and a forget gate per channel that never falls
 below a learned bound, f = l + (1 - l) sigmoid(W_f h + b); with a state S [dim, vdim] that starts at zero and ' for transposed:
