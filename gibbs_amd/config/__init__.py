@@ -6,6 +6,7 @@ from .rukosun import RukosunConfig
 from .ruzinex import RuzinexConfig
 from .litizen import LitizenConfig
 from .gumozen import GumozenConfig
+from .lubavik import LubavikConfig
 from .registry import (Architecture, architectures, config_from_dict,
                        find_architecture, register_architecture)
 from .spec import (ConnectionSpec, EmbeddingTablesSpec, FeedForwardSpec, LayerSpec, MixerSpec, ModelSpec, NormSpec,
@@ -17,3 +18,4 @@ register_architecture("Rukosun", RukosunConfig, aliases=("rukosun",))
 register_architecture("Ruzinex", RuzinexConfig, aliases=("ruzinex",))
 register_architecture("Litizen", LitizenConfig, aliases=("litizen",))
 register_architecture("Gumozen", GumozenConfig, aliases=("gumozen",))
+register_architecture("Lubavik", LubavikConfig, aliases=("lubavik",))

@@ -17,13 +17,15 @@ from typing import Any, Mapping, Optional, Sequence, Tuple, Union
 class NormSpec:
     """A normalisation over the last axis. `kind` selects the part (`"rms"`; `"layer"`: mean taken off, gain and bias;
     `"group_rms"`: the row in `groups` equal consecutive parts, each divided by its own root mean square).  `scale` names a
-    further vector per channel that multiplies the normed row (a layer scale)."""
+    further vector per channel that multiplies the normed row (a layer scale).  `offset` is added to the stored weight (1: the
+    weight is stored around zero and the gain is 1 + w)."""
     kind: str
     eps: float
     weight: str                     # tensor name of the gain
     bias: Optional[str] = None      # tensor name of the bias (kinds that have one)
     groups: int = 1                 # parts of the row that are normed by themselves (kind "group_rms")
     scale: Optional[str] = None     # tensor name of a further scale per channel (kind "rms")
+    offset: float = 0.0             # added to the stored weight (kind "rms")
 
 
 @dataclass(frozen=True)

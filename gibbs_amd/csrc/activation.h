@@ -7,6 +7,8 @@ enum { ACT_SILU = 0, ACT_GELU_TANH = 1, ACT_GELU = 2, ACT_RELU = 3, ACT_COUNT = 
 // One more code, for gated products only: the clamped variant, which is no act(gate) * up:
 //   the gate capped at `limit` from above, the up value clipped to +-limit; then gate * sigmoid(alpha * gate) * (1 + up)
 enum { ACT_CLAMPED_SWISH = 4 };
+// And one for feed-forwards without a gate: the square of relu.
+enum { ACT_RELU_SQUARED = 5 };
 __device__ __forceinline__ float clamped_swish_product(float gate, float up, float alpha, float limit) {
   const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
   return g * (1.0f / (1.0f + expf(-alpha * g))) * (u + 1.0f);
@@ -20,6 +22,7 @@ __device__ __forceinline__ float activate(float g, int act) {
     }
     case ACT_GELU: return 0.5f * g * (1.0f + erff(g * 0.7071067811865476f));
     case ACT_RELU: return fmaxf(g, 0.0f);
+    case ACT_RELU_SQUARED: { const float r = fmaxf(g, 0.0f); return r * r; }
     default: return g * (1.0f / (1.0f + expf(-g)));   // silu
   }
 }

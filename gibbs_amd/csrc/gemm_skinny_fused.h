@@ -15,7 +15,7 @@ typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 bf16x8;
 typedef __attribute__((__vector_size__(4 * sizeof(__bf16)))) __bf16 bf16x4;
 typedef __attribute__((__vector_size__(4 * sizeof(float)))) float floatx4;
 
-enum { EPI_STORE = 0, EPI_RESIDUAL = 1, EPI_GLU = 2, EPI_CONV = 3 };
+enum { EPI_STORE = 0, EPI_RESIDUAL = 1, EPI_GLU = 2, EPI_CONV = 3, EPI_ACT = 4 };
 
 // The operand with lanes r and r ^ 8 of every 16 exchanged (a rotation by 8 within the row of lanes).
 __device__ __forceinline__ bf16x8 swap_halves16(bf16x8 v) {
@@ -57,6 +57,11 @@ struct FusedArgs {
   int K;
   int act;  // GLU: the activation's code
   float act_alpha, act_limit;   // of the clamped variant (ACT_CLAMPED_SWISH)
+  // ACT: y = act(product), times the entries of the row's token in a second table (null: none), [vocab, mult_ld] from column 0 of `mult`
+  const bf16* mult;
+  long mult_ld;
+  const int* ids;   // [N]
+  int vocab;
 };
 
 // KC: the convolution's kernel length when it is 2..4 (its operands are then asked for before the
@@ -354,6 +359,11 @@ __global__ __launch_bounds__(WAVES * WAVE) void gemm_skinny_fused_kernel(const b
 #pragma unroll
     for (int i = 0; i < 4; ++i) pre_x[i] = (epi_lane && o_epi + i < a.O) ? a.x[(size_t)n_epi * a.O + o_epi + i] : 0.f;
   }
+  if (EPI == EPI_ACT && a.mult) {
+    const int id = epi_lane ? min(max(a.ids[n_epi], 0), a.vocab - 1) : 0;      // (never read outside the table)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) pre_x[i] = (epi_lane && o_epi + i < a.O) ? (float)a.mult[(size_t)id * a.mult_ld + o_epi + i] : 0.f;
+  }
   if (EPI == EPI_CONV && KC > 1) {
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
@@ -462,6 +472,13 @@ __global__ __launch_bounds__(WAVES * WAVE) void gemm_skinny_fused_kernel(const b
       } else {
         for (int i = 0; i < 4 && o + i < a.O; ++i) { xp[i] = v[i]; bp[i] = (bf16)v[i]; }
       }
+    } else if (EPI == EPI_ACT) {
+      bf16* y = a.Y + (size_t)n * a.ldy + o;
+      bf16 v[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) v[i] = (bf16)(activate(sum[0][i], a.act) * (a.mult ? pre_x[i] : 1.0f));
+      if (full && a.y_vec) *(bf16x4*)y = bf16x4{v[0], v[1], v[2], v[3]};
+      else for (int i = 0; i < 4 && o + i < a.O; ++i) y[i] = v[i];
     } else if (EPI == EPI_GLU) {
       bf16* y = a.Y + (size_t)n * a.ldy + o;
       bf16 v[4];
@@ -618,6 +635,8 @@ void run_store(const FusedArgs& a, bool rms, hipStream_t s) {
   if (rms) launch_nt<TILED, 1, true, EPI_STORE>(a, s);
   else launch_nt<TILED, 1, false, EPI_STORE>(a, s);
 }
+template <bool TILED>
+void run_act(const FusedArgs& a, hipStream_t s) { launch_nt<TILED, 1, false, EPI_ACT>(a, s); }
 template <bool TILED>
 void run_residual(const FusedArgs& a, hipStream_t s) { launch_nt<TILED, 1, false, EPI_RESIDUAL>(a, s); }
 template <bool TILED>

@@ -28,6 +28,7 @@
 //                  RESIDUAL  x += acc (float32 stream, each element owned by one workgroup);
 //                            xb = bfloat16(x), the mirror the next product reads
 //                  GLU       out = act(gate) * up (activation.h)
+//                  ACT       y = act(acc), times the token's entries of a second table
 //                  CONV      bx = B * x;  cv = bias + taps . [state, bx];  y = C * cv;  state shifts
 //                            (every row is one decoded token of a different request)
 #include "gemm_skinny_fused.h"
@@ -96,6 +97,22 @@ GIBBS_EXPORT int gibbs_skinny_glu_general(const void* X, const void* W, void* Y,
   if (a.packed) run_glu<true>(a, rms != 0, stream);
   else gibbs_fused_rows(&a, EPI_GLU, rms, stream);
   GIBBS_LAUNCH_STATUS("skinny_glu");
+}
+
+// out[n, o] = act(W_o . X_n) (* table[id_n, o]); table: bfloat16 rows of mult_ld values, or null.
+GIBBS_EXPORT int gibbs_skinny_act(const void* X, const void* W, void* Y, int N, int O, int I, long ldx, long ldw, long ldy, int act,
+                                  const void* mult, long mult_ld, const int* ids, int vocab, hipStream_t stream) {
+  if (check_common("skinny_act", X, W, N, O, I, ldx, ldw)) return 1;
+  GIBBS_REQUIRE(ldy >= O, "skinny_act: output rows shorter than %d", O);
+  GIBBS_REQUIRE((act >= 0 && act < ACT_COUNT) || act == ACT_RELU_SQUARED, "skinny_act: unknown activation %d", act);
+  GIBBS_REQUIRE(!mult || (ids && vocab > 0 && mult_ld >= O), "skinny_act: a table without the rows' tokens, or rows of %ld entries", mult_ld);
+  FusedArgs a{};
+  a.W = (const bf16*)W; a.X = (const bf16*)X; a.N = N; a.O = O; a.I = I; a.ldw = ldw; a.ldx = ldx; note_layout(a);
+  a.Y = (bf16*)Y; a.ldy = ldy; a.act = act; a.mult = (const bf16*)mult; a.mult_ld = mult_ld; a.ids = ids; a.vocab = vocab;
+  a.y_vec = ldy % 4 == 0 && ((uintptr_t)Y % 8) == 0;
+  if (a.packed) run_act<true>(a, stream);
+  else gibbs_fused_rows(&a, EPI_ACT, 0, stream);
+  GIBBS_LAUNCH_STATUS("skinny_act");
 }
 
 // In-projection and gated short convolution of N decoded tokens of N different requests:

@@ -8,6 +8,7 @@ void gibbs_fused_rows(const void* args, int epilogue, int rms, hipStream_t strea
   switch (epilogue) {
     case EPI_STORE: run_store<false>(a, rms != 0, stream); break;
     case EPI_RESIDUAL: run_residual<false>(a, stream); break;
+    case EPI_ACT: run_act<false>(a, stream); break;
     case EPI_GLU: run_glu<false>(a, rms != 0, stream); break;
     default: run_conv<false>(a, rms != 0, stream); break;
   }

@@ -119,7 +119,47 @@ int gibbs_gated_outer_step(const void* raw, long ld, int dtype, const float* bia
                            float* state, long slot_stride, const int* slot, void* out, int n_req, int H, int D, int V, hipStream_t stream);
 int gibbs_gated_outer_rule(const float* q, const float* k, const float* v, const float* decay, float* state, long slot_stride,
                            const int* cu, const int* slot, float* out, int n_req, int H, int D, int V, hipStream_t stream);
+// ---- gated_linear.hip: gated linear attention (kernels in gated_rule.h)
+int gibbs_gated_linear_rows_take(int D, int V);
+int gibbs_gated_linear_chunks_take(int D, int V);
+long gibbs_gated_linear_chunks_workspace(int rows, int n_req, int H, int D, int V);
+int gibbs_gated_linear_rows(const void* raw, long ld, int off_q, int off_k, int off_v, int off_g, int off_z, const void* w_z, int rank,
+                            const float* bias, float inv_tau, float q_scale, const float* gain, float eps, float* state, long slot_stride,
+                            const int* cu, const int* slot, void* out, int dtype, int n_req, int H, int D, int V, hipStream_t stream);
+int gibbs_gated_linear_chunks(const void* raw, long ld, int off_q, int off_k, int off_v, int off_g, const float* z, const float* bias,
+                              float inv_tau, float q_scale, const float* gain, float eps, float* state, long slot_stride, const int* cu,
+                              const int* slot, void* out, float* workspace, int dtype, int n_rows, int n_req, int H, int D, int V,
+                              hipStream_t stream);
+// ---- matrix_lstm.hip: matrix memory with exponential gates and a normaliser
+int gibbs_matrix_lstm_rows_take(int D, int V);
+int gibbs_matrix_lstm_chunks_take(int D, int V);
+long gibbs_matrix_lstm_chunks_workspace(int rows, int n_req, int H, int D, int V);
+int gibbs_matrix_lstm_rows(const void* raw, long ld, int off_q, int off_k, int off_v, int off_g, const void* h, int W, const void* w_gates,
+                           const float* b_gates, const float* gain, float cap, float eps, float q_scale, float* state, float* norm_state,
+                           long slot_stride, const int* cu, const int* slot, void* out, int dtype, int n_req, int H, int D, int V,
+                           hipStream_t stream);
+int gibbs_matrix_lstm_chunks(const void* raw, long ld, int off_q, int off_k, int off_v, int off_g, const void* h, int W, const void* w_gates,
+                             const float* b_gates, const float* gain, float cap, float eps, float q_scale, float* state, float* norm_state,
+                             long slot_stride, const int* cu, const int* slot, void* out, const float* gates, float* workspace, int dtype,
+                             int n_rows, int n_req, int H, int D, int V, hipStream_t stream);
+// ---- rows of a feed-forward without a gate; a norm over the whole projection; sums of two results at a sublayer's boundary
+int gibbs_act_rows(const void* z, void* out, long ld_out, int dtype, int act, const void* mult, long mult_ld, const int* ids, int vocab,
+                   int n_rows, int F, hipStream_t stream);
+int gibbs_skinny_act(const void* X, const void* W, void* Y, int N, int O, int I, long ldx, long ldw, long ldy, int act, const void* mult,
+                     long mult_ld, const int* ids, int vocab, hipStream_t stream);
+int gibbs_qkv_prepare_whole(void* rows, long ld, void* kpages, void* vpages, int dtype, const float* q_gain, const float* k_gain, float eps,
+                            int norm_dim, const float* inv_freq, int rot, int variant, const float* cs_table, int table_len, const int* pos,
+                            const int* row_req, const int* table, int max_pages, int page_size, int num_pages, int n_rows, int nh, int nkv,
+                            int hd, int vd, hipStream_t stream);
+int gibbs_rmsnorm_rows_sum_add_read(float* x, const void* in, int parts, long part_stride, const float* bias, float scale, const void* in2,
+                                    int parts2, float scale2, const float* gain, float eps, int read, void* out, int dtype, int n,
+                                    int hidden, hipStream_t stream);
+int gibbs_rows_terms(const void* in, int parts, const float* bias, float scale, const void* in2, int parts2, float scale2, float* out,
+                     int dtype, int n, int hidden, hipStream_t stream);
 // ---- moe.hip: mixture of experts
+int gibbs_moe_route_scaled(const void* h, long ldh, int dtype, const float* router, const float* router_bias, const float* shared_gate,
+                           int* chosen, float* weight, float* sgate, int n, int W, int E, int top, int mode, float weight_scale,
+                           hipStream_t stream);
 long gibbs_moe_capacity(int n_pairs, int E, int bm);
 int gibbs_moe_tile(int n_pairs, int E);
 int gibbs_moe_route(const void* h, long ldh, int dtype, const float* router, const float* router_bias, const float* shared_gate,

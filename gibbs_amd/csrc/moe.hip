@@ -4,7 +4,7 @@
 //   route      z = W_r h + b in float32 (h as the step holds it); the `top` largest logits (the lower index among
 //              equals); weights = softmax over the chosen logits alone; gate = sigmoid(w_sg . h) for the shared expert
 //              (mode 1: scores s = softmax(z) over all router outputs; the `top` largest of s + correction; weights = the
-//              chosen scores s divided by their sum + 1e-20; mode 2: scores s = sigmoid(z), the `top` largest of s +
+//              chosen scores s divided by their sum + 1e-20, times a constant; mode 2: scores s = sigmoid(z), the `top` largest of s +
 //              correction, or of z without one, weights = the chosen scores s as they are.  Router outputs from `E_real` on are identity experts: they
 //              have no matrices, their result is the row itself, and their pairs take no place in the tiles)
 //   group      the step's (row, choice) pairs sorted by expert into tiles of `bm` pairs that belong to one expert
@@ -111,7 +111,7 @@ template <typename T>
 __global__ __launch_bounds__(1024) void moe_route_kernel(const T* __restrict__ h, long ldh, const float* __restrict__ router,
                                                         const float* __restrict__ router_bias, const float* __restrict__ shared_gate,
                                                         int* __restrict__ chosen, float* __restrict__ weight, float* __restrict__ sgate,
-                                                        int W, int E, int top, int mode) {
+                                                        int W, int E, int top, int mode, float weight_scale) {
   extern __shared__ float z[];   // [E] (mode 1 and 2: and the scores behind them, [E])
   const int n = blockIdx.x, wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE, n_waves = blockDim.x / WAVE;
   const T* row = h + (size_t)n * ldh;
@@ -204,7 +204,7 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(const T* __restrict__ h
   }
   if (lane == 0 && mode != 2) {
     if (mode == 1)
-      for (int c = 0; c < top; ++c) wts[c] = wts[c] / (sum + 1e-20f);
+      for (int c = 0; c < top; ++c) wts[c] = wts[c] / (sum + 1e-20f) * weight_scale;
     else
       for (int c = 0; c < top; ++c) wts[c] = sum > 0.f ? wts[c] / sum : 0.f;
   }
@@ -625,9 +625,11 @@ GIBBS_EXPORT int gibbs_moe_tile(int n_pairs, int E) { return (long)n_pairs <= 64
 // mode 0: the largest logits (+ bias), weights by the softmax over the chosen; mode 1: scores by the softmax over all E
 // outputs, the largest of score + router_bias (a correction that only the choice sees), weights the chosen scores over their sum;
 // mode 2: scores by the sigmoid of every output alone, the largest of score + router_bias, weights the chosen scores.
-GIBBS_EXPORT int gibbs_moe_route_mode(const void* h, long ldh, int dtype, const float* router, const float* router_bias,
-                                      const float* shared_gate, int* chosen, float* weight, float* sgate, int n, int W, int E, int top,
-                                      int mode, hipStream_t stream) {
+// weight_scale: mode 1's weights times a constant.
+GIBBS_EXPORT int gibbs_moe_route_scaled(const void* h, long ldh, int dtype, const float* router, const float* router_bias,
+                                        const float* shared_gate, int* chosen, float* weight, float* sgate, int n, int W, int E, int top,
+                                        int mode, float weight_scale, hipStream_t stream) {
+  GIBBS_REQUIRE(weight_scale == 1.0f || mode == 1, "moe_route: weights times %g go with the scores' softmax over all outputs", weight_scale);
   GIBBS_REQUIRE(mode >= 0 && mode <= 2, "moe_route: mode %d", mode);
   GIBBS_REQUIRE(h && router && chosen && weight && n > 0 && W > 0 && ldh >= W, "moe_route: bad operands n=%d width=%d", n, W);
   GIBBS_REQUIRE(E > 0 && E <= MOE_MAX_EXPERTS && top > 0 && top <= E, "moe_route: %d of %d experts (at most %d)", top, E, MOE_MAX_EXPERTS);
@@ -636,12 +638,17 @@ GIBBS_EXPORT int gibbs_moe_route_mode(const void* h, long ldh, int dtype, const 
   // few rows: a wave per expert (and one for the shared expert's gate) up to 16 waves; many rows fill the chip with 4
   const int threads = n >= 512 ? 256 : WAVE * std::min(16, std::max(4, E + 1));
   if (dtype == GIBBS_F32)
-    moe_route_kernel<float><<<n, threads, lds, stream>>>((const float*)h, ldh, router, router_bias, shared_gate, chosen, weight, sgate, W, E, top, mode);
+    moe_route_kernel<float><<<n, threads, lds, stream>>>((const float*)h, ldh, router, router_bias, shared_gate, chosen, weight, sgate, W, E, top, mode, weight_scale);
   else if (dtype == GIBBS_BF16)
-    moe_route_kernel<bf16><<<n, threads, lds, stream>>>((const bf16*)h, ldh, router, router_bias, shared_gate, chosen, weight, sgate, W, E, top, mode);
+    moe_route_kernel<bf16><<<n, threads, lds, stream>>>((const bf16*)h, ldh, router, router_bias, shared_gate, chosen, weight, sgate, W, E, top, mode, weight_scale);
   else
     return gibbs_fail("moe_route: unknown dtype %d", dtype);
   GIBBS_LAUNCH_STATUS("moe_route");
+}
+GIBBS_EXPORT int gibbs_moe_route_mode(const void* h, long ldh, int dtype, const float* router, const float* router_bias,
+                                      const float* shared_gate, int* chosen, float* weight, float* sgate, int n, int W, int E, int top,
+                                      int mode, hipStream_t stream) {
+  return gibbs_moe_route_scaled(h, ldh, dtype, router, router_bias, shared_gate, chosen, weight, sgate, n, W, E, top, mode, 1.0f, stream);
 }
 GIBBS_EXPORT int gibbs_moe_route(const void* h, long ldh, int dtype, const float* router, const float* router_bias,
                                  const float* shared_gate, int* chosen, float* weight, float* sgate, int n, int W, int E, int top,

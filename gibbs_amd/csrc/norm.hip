@@ -259,6 +259,8 @@ __global__ void rmsnorm_rows_add_kernel(float* __restrict__ x, const void* __res
 // MIX: the part's result is itself a weighted sum that no kernel has written yet (a mixture of experts' combination):
 // v = sum_s weight[n][s] * in[place[n][s]] (ascending s, rows of `in` in the activation type) + gate[n] * shared[n]
 // (shared null: none; gate or weight null: 1), float32 throughout.
+// SUM: the result is a sum of two sublayers' results side by side, or has a bias per channel: v = scale (in + bias) + scale2 in2, each of
+// the two as partial sums or in the activation type (in2 or bias null: none).
 // READ: what `out` takes of the new x: READ_NORM its norm (above), READ_ROWS the row as it is (a sublayer that is not normed on
 // its way in), READ_SHIFT the row mixed with the request's previous one, x + (before - x) mu, in a step where every request
 // brings one row: before is the request's state, which the row replaces.
@@ -276,10 +278,29 @@ struct RowMix {
   const float* gate;      // [n] or null
   int top;
 };
-template <typename T, int CHUNKS, bool MIX, int READ>
+struct RowSum {
+  const float* bias;      // [hidden] or null
+  float scale;
+  const void* in2;        // null: none
+  int parts2;
+  float scale2;
+};
+enum { FROM_ROWS = 0, FROM_MIX = 1, FROM_SUM = 2 };
+template <typename T>
+__device__ __forceinline__ float4 sum_parts4(const void* in, int parts, size_t part_stride, size_t i) {
+  if (parts == 1) return load4((const T*)in + i);
+  float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+  for (int s = 0; s < parts; ++s) {
+    const float4 d = *(const float4*)((const float*)in + s * part_stride + i);
+    v.x += d.x; v.y += d.y; v.z += d.z; v.w += d.w;
+  }
+  return v;
+}
+template <typename T, int CHUNKS, int FROM, int READ>
 __global__ void rows_add_norm_vec_kernel(float* __restrict__ x, const void* __restrict__ in, int parts, size_t part_stride,
                                          const float* __restrict__ gain_d, float eps_d, const float* __restrict__ gain_n, float eps_n,
-                                         T* __restrict__ out, int hidden, RowMix mix, RowShift shift) {
+                                         T* __restrict__ out, int hidden, RowMix mix, RowShift shift, RowSum sum) {
+  constexpr bool MIX = FROM == FROM_MIX;
   __shared__ float scratch[16];
   const size_t at = (size_t)blockIdx.x * hidden;
   float4 v[CHUNKS], xv[CHUNKS], before[READ == READ_SHIFT ? CHUNKS : 1];
@@ -305,12 +326,19 @@ __global__ void rows_add_norm_vec_kernel(float* __restrict__ x, const void* __re
           const float4 r = load4((const T*)mix.shared + at + i);
           v[c].x = fmaf(g, r.x, v[c].x); v[c].y = fmaf(g, r.y, v[c].y); v[c].z = fmaf(g, r.z, v[c].z); v[c].w = fmaf(g, r.w, v[c].w);
         }
-      } else if (parts == 1) {
-        v[c] = load4((const T*)in + at + i);
       } else {
-        for (int s = 0; s < parts; ++s) {
-          const float4 d = *(const float4*)((const float*)in + s * part_stride + at + i);
-          v[c].x += d.x; v[c].y += d.y; v[c].z += d.z; v[c].w += d.w;
+        v[c] = sum_parts4<T>(in, parts, part_stride, at + i);
+        if constexpr (FROM == FROM_SUM) {
+          if (sum.bias) {
+            const float4 b = *(const float4*)(sum.bias + i);
+            v[c].x += b.x; v[c].y += b.y; v[c].z += b.z; v[c].w += b.w;
+          }
+          v[c].x *= sum.scale; v[c].y *= sum.scale; v[c].z *= sum.scale; v[c].w *= sum.scale;
+          if (sum.in2) {
+            const float4 d = sum_parts4<T>(sum.in2, sum.parts2, part_stride, at + i);
+            v[c].x = fmaf(sum.scale2, d.x, v[c].x); v[c].y = fmaf(sum.scale2, d.y, v[c].y);
+            v[c].z = fmaf(sum.scale2, d.z, v[c].z); v[c].w = fmaf(sum.scale2, d.w, v[c].w);
+          }
         }
       }
       ss += v[c].x * v[c].x + v[c].y * v[c].y + v[c].z * v[c].z + v[c].w * v[c].w;
@@ -354,7 +382,7 @@ __global__ void rows_add_norm_vec_kernel(float* __restrict__ x, const void* __re
 template <typename T>
 bool launch_rows_add_norm(float* x, const void* in, int parts, long part_stride, const float* gain_d, float eps_d, const float* gain_n,
                           float eps_n, T* out, int n, int hidden, hipStream_t stream, const RowMix* mixed = nullptr, int read = READ_NORM,
-                          const RowShift& shift = RowShift{}) {
+                          const RowShift& shift = RowShift{}, const RowSum* summed = nullptr) {
   const uintptr_t vec = parts == 1 ? 4 * sizeof(T) : 16;
   if (hidden % 4 || ((uintptr_t)x % 16) || ((uintptr_t)in % vec) || (parts > 1 && part_stride % 4) || (gain_d && ((uintptr_t)gain_d % 16)) ||
       (gain_n && ((uintptr_t)gain_n % 16)) || (out && ((uintptr_t)out % (4 * sizeof(T)))) ||
@@ -365,18 +393,26 @@ bool launch_rows_add_norm(float* x, const void* in, int parts, long part_stride,
   const int chunks = ceil_div(hidden, 4 * threads);
   if (read == READ_SHIFT && (shift.slot_stride % 4 || ((uintptr_t)shift.state % 16) || ((uintptr_t)shift.mu % 16))) return false;
   const RowMix mix = mixed ? *mixed : RowMix{};
+  const RowSum sum = summed ? *summed : RowSum{};
+  if (summed) {
+    const uintptr_t vec2 = summed->parts2 == 1 ? 4 * sizeof(T) : 16;
+    if (((uintptr_t)summed->bias % 16) || (summed->in2 && ((uintptr_t)summed->in2 % vec2)) || part_stride % 4 || mixed || read == READ_SHIFT) return false;
+  }
 #define GIBBS_ROWS_ADD_READ(C, M, R) \
-  rows_add_norm_vec_kernel<T, C, M, R><<<n, threads, 0, stream>>>(x, in, parts, (size_t)part_stride, gain_d, eps_d, gain_n, eps_n, out, hidden, mix, shift)
+  rows_add_norm_vec_kernel<T, C, M, R><<<n, threads, 0, stream>>>(x, in, parts, (size_t)part_stride, gain_d, eps_d, gain_n, eps_n, out, hidden, mix, shift, sum)
 #define GIBBS_ROWS_ADD_NORM(C)                                                                     \
   do {                                                                                             \
     if (mixed) {                                                                                   \
-      if (read == READ_SHIFT) GIBBS_ROWS_ADD_READ(C, true, READ_SHIFT);                            \
-      else if (read == READ_ROWS) GIBBS_ROWS_ADD_READ(C, true, READ_ROWS);                         \
-      else GIBBS_ROWS_ADD_READ(C, true, READ_NORM);                                                \
+      if (read == READ_SHIFT) GIBBS_ROWS_ADD_READ(C, FROM_MIX, READ_SHIFT);                        \
+      else if (read == READ_ROWS) GIBBS_ROWS_ADD_READ(C, FROM_MIX, READ_ROWS);                     \
+      else GIBBS_ROWS_ADD_READ(C, FROM_MIX, READ_NORM);                                            \
+    } else if (summed) {                                                                           \
+      if (read == READ_ROWS) GIBBS_ROWS_ADD_READ(C, FROM_SUM, READ_ROWS);                          \
+      else GIBBS_ROWS_ADD_READ(C, FROM_SUM, READ_NORM);                                            \
     } else {                                                                                       \
-      if (read == READ_SHIFT) GIBBS_ROWS_ADD_READ(C, false, READ_SHIFT);                           \
-      else if (read == READ_ROWS) GIBBS_ROWS_ADD_READ(C, false, READ_ROWS);                        \
-      else GIBBS_ROWS_ADD_READ(C, false, READ_NORM);                                               \
+      if (read == READ_SHIFT) GIBBS_ROWS_ADD_READ(C, FROM_ROWS, READ_SHIFT);                       \
+      else if (read == READ_ROWS) GIBBS_ROWS_ADD_READ(C, FROM_ROWS, READ_ROWS);                    \
+      else GIBBS_ROWS_ADD_READ(C, FROM_ROWS, READ_NORM);                                           \
     }                                                                                              \
   } while (0)
   if (chunks == 1) GIBBS_ROWS_ADD_NORM(1);
@@ -438,6 +474,51 @@ GIBBS_EXPORT int gibbs_rmsnorm_rows_add_read(float* x, const void* in, int parts
   else return gibbs_fail("rmsnorm_rows_add_read: unknown dtype %d", dtype);
   if (!queued) return -1;
   GIBBS_LAUNCH_STATUS("rmsnorm_rows_add_read");
+}
+
+// The same with v = scale (in + bias) + scale2 in2 (bias [hidden] or in2 null: none; partial sums of both lie part_stride apart), and read
+// 0 nothing or 1 the rows of the new x.
+GIBBS_EXPORT int gibbs_rmsnorm_rows_sum_add_read(float* x, const void* in, int parts, long part_stride, const float* bias, float scale, const void* in2,
+                                                 int parts2, float scale2, const float* gain, float eps, int read, void* out, int dtype, int n,
+                                                 int hidden, hipStream_t stream) {
+  GIBBS_REQUIRE(x && in && n >= 0 && hidden > 0 && parts >= 1 && (!in2 || parts2 >= 1), "rmsnorm_rows_sum_add_read: bad sizes n=%d hidden=%d parts=%d, %d", n, hidden, parts, parts2);
+  GIBBS_REQUIRE((read == 0 || read == 1) && (read == 0 || out), "rmsnorm_rows_sum_add_read: bad reader %d", read);
+  if (n == 0) return 0;
+  const RowSum sum{bias, scale, in2, parts2, scale2};
+  void* o = read ? out : nullptr;
+  bool queued;
+  if (dtype == GIBBS_F32) queued = launch_rows_add_norm<float>(x, in, parts, part_stride, gain, eps, nullptr, 0.f, (float*)o, n, hidden, stream, nullptr, read, RowShift{}, &sum);
+  else if (dtype == GIBBS_BF16) queued = launch_rows_add_norm<bf16>(x, in, parts, part_stride, gain, eps, nullptr, 0.f, (bf16*)o, n, hidden, stream, nullptr, read, RowShift{}, &sum);
+  else return gibbs_fail("rmsnorm_rows_sum_add_read: unknown dtype %d", dtype);
+  if (!queued) return -1;
+  GIBBS_LAUNCH_STATUS("rmsnorm_rows_sum_add_read");
+}
+
+// The terms of such a sum as two float32 partial sums, out [2, n, hidden]: scale (in + bias) and scale2 in2 (zeros without), for whoever
+// takes partial sums only.
+template <typename T>
+__global__ void rows_terms_kernel(const void* __restrict__ in, int parts, const float* __restrict__ bias, float scale, const void* __restrict__ in2,
+                                  int parts2, float scale2, float* __restrict__ out, size_t count, int hidden) {
+  const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= count) return;
+  auto total = [&](const void* p, int k) -> float {
+    if (k == 1) return to_float(((const T*)p)[i]);
+    float v = 0.f;
+    for (int s = 0; s < k; ++s) v += ((const float*)p)[s * count + i];
+    return v;
+  };
+  out[i] = scale * (total(in, parts) + (bias ? bias[i % hidden] : 0.f));
+  out[count + i] = in2 ? scale2 * total(in2, parts2) : 0.f;
+}
+GIBBS_EXPORT int gibbs_rows_terms(const void* in, int parts, const float* bias, float scale, const void* in2, int parts2, float scale2, float* out,
+                                  int dtype, int n, int hidden, hipStream_t stream) {
+  GIBBS_REQUIRE(in && out && n >= 0 && hidden > 0 && parts >= 1 && (!in2 || parts2 >= 1), "rows_terms: bad sizes n=%d hidden=%d", n, hidden);
+  if (n == 0) return 0;
+  const long count = (long)n * hidden;
+  if (dtype == GIBBS_F32) rows_terms_kernel<float><<<ceil_div(count, 256), 256, 0, stream>>>(in, parts, bias, scale, in2, parts2, scale2, out, (size_t)count, hidden);
+  else if (dtype == GIBBS_BF16) rows_terms_kernel<bf16><<<ceil_div(count, 256), 256, 0, stream>>>(in, parts, bias, scale, in2, parts2, scale2, out, (size_t)count, hidden);
+  else return gibbs_fail("rows_terms: unknown dtype %d", dtype);
+  GIBBS_LAUNCH_STATUS("rows_terms");
 }
 
 GIBBS_EXPORT int gibbs_rmsnorm_rows_add(float* x, const void* in, int parts, long part_stride, const float* gain, float eps, int dtype,

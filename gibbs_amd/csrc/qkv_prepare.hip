@@ -21,6 +21,7 @@
 // unnormed, unrotated key into the value page); and values turned by their position over all of their first `v_rot`
 // channels, pairs in the same layout, angle float(pos) * v_inv_freq[m], before they are cached.  `gibbs_attention_finish`
 // is the other end of that: the heads' outputs turned back by the query's position and multiplied by sigmoid(gate).
+// `gibbs_qkv_prepare_whole` is the preparation with a norm over the whole projection of q (and of k) instead of one per head.
 #include "common.h"
 #include "lane8.h"
 
@@ -271,6 +272,90 @@ __global__ __launch_bounds__(256) void attention_finish_kernel(T* __restrict__ a
   if (g)
     for (int e = 2 * vh + lane; e < vd; e += WAVE) o[e] = from_float<T>(gated(e, to_float(o[e])));
 }
+// q and k divided by the root mean square of the WHOLE projection (all heads of q at once, all heads of k at once) and multiplied by a
+// gain per stored channel, before the rotation: a workgroup per row.  The row's q and k wait in LDS as float32 between the sums and the
+// rotation, so that a channel finds its partner whichever thread loaded it.  V: channels a thread takes at a time (8: 16-byte
+// accesses; sizes, offsets and the rotated part in steps of 8, the pairs of half-split rotations in steps of 8 as well).  nkv 0: the
+// mixer reads another layer's pages, rows are [q].
+template <typename T, int V>
+__global__ __launch_bounds__(256) void qkv_prepare_whole_kernel(T* __restrict__ rows, T* __restrict__ kpages, T* __restrict__ vpages, QkvPrepareArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float buf[];      // [(nh + nkv) hd]
+  __shared__ float scratch_q[16], scratch_k[16];
+  const int n = blockIdx.x, nq = a.nh * a.hd, nk = a.nkv * a.hd, half = a.inv_freq ? a.rot / 2 : 0;
+  T* row = rows + (size_t)n * a.ld;
+  auto load = [&](const T* p, float* f) {
+    if constexpr (V == 8 && sizeof(T) == 2) unpack_bf16x8(*(const uint4*)p, f);
+    else if constexpr (V == 8) {
+      const float4 x = *(const float4*)p, y = *(const float4*)(p + 4);
+      f[0] = x.x; f[1] = x.y; f[2] = x.z; f[3] = x.w; f[4] = y.x; f[5] = y.y; f[6] = y.z; f[7] = y.w;
+    } else f[0] = to_float(*p);
+  };
+  auto store = [&](T* p, const float* f) {
+    if constexpr (V == 8 && sizeof(T) == 2) *(uint4*)p = pack_bf16x8(f);
+    else if constexpr (V == 8) { *(float4*)p = make_float4(f[0], f[1], f[2], f[3]); *(float4*)(p + 4) = make_float4(f[4], f[5], f[6], f[7]); }
+    else *p = from_float<T>(f[0]);
+  };
+  float ssq = 0.f, ssk = 0.f;
+  for (int e = threadIdx.x * V; e < nq + nk; e += blockDim.x * V) {
+    float f[V];
+    load(row + e, f);
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < V; ++i) {
+      buf[e + i] = f[i];
+      ss = fmaf(f[i], f[i], ss);
+    }
+    if (e < nq) ssq += ss; else ssk += ss;
+  }
+  ssq = block_sum(ssq, scratch_q);
+  ssk = block_sum(ssk, scratch_k);               // (the barriers inside publish buf as well)
+  // (heads stored wider than they are have zeros behind: the mean counts the true channels)
+  const float inv_q = 1.0f / sqrtf(ssq / (float)(a.nh * a.norm_dim) + a.qk_eps);
+  const float inv_k = nk ? 1.0f / sqrtf(ssk / (float)(a.nkv * a.norm_dim) + a.qk_eps) : 0.f;
+  const int p = a.pos[n];
+  int page = -1, at = 0;
+  if (nk && kpages) {
+    page = a.table[(size_t)a.row_req[n] * a.max_pages + p / a.page_size];
+    at = p % a.page_size;
+    if (page >= a.num_pages) page = -1;          // (the host never asks for another; never write outside the pool)
+  }
+  for (int e = threadIdx.x * V; e < nq + nk; e += blockDim.x * V) {
+    const bool is_q = e < nq;
+    const int rel = is_q ? e : e - nq, head = rel / a.hd, c = rel % a.hd;
+    const float inv = is_q ? inv_q : inv_k;
+    const float* gain = is_q ? a.q_gain + rel : a.k_gain + rel;
+    float f[V];
+#pragma unroll
+    for (int i = 0; i < V; ++i) {
+      const int ch = c + i;
+      float x = buf[e + i] * inv * gain[i];
+      if (ch < 2 * half) {
+        const int j = a.variant == ROPE_HALF_SPLIT ? (ch < half ? ch : ch - half) : ch / 2;
+        const bool first = a.variant == ROPE_HALF_SPLIT ? ch < half : (ch & 1) == 0;
+        const int step = a.variant == ROPE_HALF_SPLIT ? (first ? half : -half) : (first ? 1 : -1);
+        const float y = buf[e + i + step] * inv * gain[i + step];
+        float cs, sn;
+        if (a.cs_table && p < a.table_len) {
+          const float2 t = a.cs_table[(size_t)p * half + j];
+          cs = t.x;
+          sn = t.y;
+        } else {
+          rope_cos_sin((float)p * a.inv_freq[j], &cs, &sn);
+        }
+        x = first ? x * cs - y * sn : x * cs + y * sn;
+      }
+      f[i] = x;
+    }
+    store(row + e, f);
+    if (!is_q && page >= 0) store(kpages + (((size_t)page * a.nkv + head) * a.page_size + at) * a.hd + c, f);
+  }
+  if (page < 0) return;
+  for (int e = threadIdx.x * V; e < a.nkv * a.vd; e += blockDim.x * V) {
+    float f[V];
+    load(row + nq + nk + e, f);
+    store(vpages + (((size_t)page * a.nkv + e / a.vd) * a.page_size + at) * a.vd + e % a.vd, f);
+  }
+}
 }  // namespace
 
 // keep_mode: 0 none, 1 the values are published into `keep`, 2 `keep` is mixed into the values with *lambda.
@@ -325,6 +410,41 @@ GIBBS_EXPORT int gibbs_qkv_prepare(void* rows, long ld, void* kpages, void* vpag
   return gibbs_qkv_prepare_full(rows, ld, kpages, vpages, dtype, bias, inv_freq, rot, variant, cs_table, table_len, keep, keep_mode, vt, lambda,
                                 pos, row_req, table, max_pages, page_size, num_pages, n_rows, nh, nkv, hd, vd, nullptr, nullptr, 0.f, 0, 0,
                                 nullptr, 0, stream);
+}
+
+// Rows [q: nh*hd | k: nkv*hd | v: nkv*vd] (nkv 0: only q): q and k normed over the whole projection (mean over heads * norm_dim channels,
+// gains [nh*hd] and [nkv*hd] in the stored layout), the first `rot` channels of every head turned, k and v into their pages.
+GIBBS_EXPORT int gibbs_qkv_prepare_whole(void* rows, long ld, void* kpages, void* vpages, int dtype, const float* q_gain, const float* k_gain,
+                                         float eps, int norm_dim, const float* inv_freq, int rot, int variant, const float* cs_table,
+                                         int table_len, const int* pos, const int* row_req, const int* table, int max_pages, int page_size,
+                                         int num_pages, int n_rows, int nh, int nkv, int hd, int vd, hipStream_t stream) {
+  GIBBS_REQUIRE(rows && pos && q_gain && (nkv == 0 || k_gain) && n_rows > 0 && nh > 0 && nkv >= 0 && hd > 0 && vd > 0 && norm_dim > 0 && norm_dim <= hd,
+                "qkv_prepare_whole: bad operands rows=%d heads=%d kv=%d", n_rows, nh, nkv);
+  GIBBS_REQUIRE(ld >= (long)(nh + nkv) * hd + (long)nkv * vd, "qkv_prepare_whole: rows of %ld values cannot hold q, k and v", ld);
+  GIBBS_REQUIRE(!kpages || (vpages && row_req && table && max_pages > 0 && page_size > 0 && num_pages > 0), "qkv_prepare_whole: pages without their table");
+  GIBBS_REQUIRE(!inv_freq || (rot > 0 && rot % 2 == 0 && rot <= hd), "qkv_prepare_whole: %d rotated channels of a head of %d", rot, hd);
+  GIBBS_REQUIRE(dtype == GIBBS_F32 || dtype == GIBBS_BF16, "qkv_prepare_whole: unknown dtype %d", dtype);
+  const size_t lds = (size_t)(nh + nkv) * hd * sizeof(float);
+  GIBBS_REQUIRE(lds <= 150 * 1024, "qkv_prepare_whole: q and k of %zu channels a row", lds / sizeof(float));
+  QkvPrepareArgs a{};
+  a.inv_freq = inv_freq; a.rot = inv_freq ? rot : 0; a.variant = variant; a.cs_table = (const float2*)cs_table; a.table_len = cs_table && inv_freq ? table_len : 0;
+  a.pos = pos; a.row_req = row_req; a.table = table; a.max_pages = max_pages; a.page_size = page_size; a.num_pages = num_pages;
+  a.nh = nh; a.nkv = nkv; a.hd = hd; a.vd = vd; a.ld = ld; a.q_gain = q_gain; a.k_gain = k_gain; a.qk_eps = eps; a.norm_dim = norm_dim;
+  const bool x8 = hd % 8 == 0 && vd % 8 == 0 && ld % 8 == 0 && ((uintptr_t)rows % 16) == 0 && (!kpages || (((uintptr_t)kpages % 16) == 0 && ((uintptr_t)vpages % 16) == 0));
+#define PREPARE_WHOLE(T, V)                                                                                                              \
+  do {                                                                                                                                   \
+    static bool raised = false;                                                                                                          \
+    if (!raised && lds > 48 * 1024) {                                                                                                    \
+      if (hipFuncSetAttribute((const void*)qkv_prepare_whole_kernel<T, V>, hipFuncAttributeMaxDynamicSharedMemorySize, 150 * 1024) != hipSuccess) \
+        return gibbs_fail("qkv_prepare_whole: the kernel's LDS could not be reserved");                                                  \
+      raised = true;                                                                                                                     \
+    }                                                                                                                                    \
+    qkv_prepare_whole_kernel<T, V><<<n_rows, 256, lds, stream>>>((T*)rows, (T*)kpages, (T*)vpages, a);                                    \
+  } while (0)
+  if (dtype == GIBBS_F32) { if (x8) PREPARE_WHOLE(float, 8); else PREPARE_WHOLE(float, 1); }
+  else { if (x8) PREPARE_WHOLE(bf16, 8); else PREPARE_WHOLE(bf16, 1); }
+#undef PREPARE_WHOLE
+  GIBBS_LAUNCH_STATUS("qkv_prepare_whole");
 }
 
 GIBBS_EXPORT int gibbs_attention_finish(void* att, long ldo, const void* gate, long ld_gate, int gate_head, int dtype, const int* pos,

@@ -49,6 +49,7 @@ constexpr int SKINNY_ROWS_F32_OUT = 48;   // the same for float32 output (the he
 constexpr int ACT_CLAMPED = 4;            // the gated feed-forward's clamped activation (activation.h: ACT_CLAMPED_SWISH)
 constexpr int SSD_CHUNKED_ROWS = 256;     // rows of one request from which the state-space rule runs in chunks
 constexpr int GATED_CHUNKED_ROWS = 96;    // rows of a request from which the gated outer-product rule runs in chunks
+constexpr int WALKED_ROWS = 24;           // rows of a request from which gated linear attention and the matrix memory run in chunks
 constexpr int MATRIX_SLICE_PAGES = 510;   // page ids of a key slice that the decode attention's matrix-core walk keeps in LDS
 
 // Ranges of k that the few-row product is cut into so that at least `want_blocks` workgroups run (a
@@ -202,10 +203,17 @@ struct Arena {
   }
 };
 
-// A delta that has not been added to the residual stream yet.
+// A delta that has not been added to the residual stream yet.  It may be a sum still to be taken: scale (data + bias) + scale2 data2 (a
+// sublayer's boundary takes it on its way; Exec::plain makes it partial sums for everyone else).
 struct Pending {
   void* data = nullptr;
   int parts = 0;   // 0: nothing; 1: [N, H] in the activation type; >= 2: float32 partial sums [parts, N, H]
+  const float* bias = nullptr;   // [H]
+  float scale = 1.f;
+  void* data2 = nullptr;         // null: no second term
+  int parts2 = 0;
+  float scale2 = 1.f;
+  bool is_plain() const { return !bias && scale == 1.f && !data2; }
 };
 
 struct Plan;
@@ -264,6 +272,8 @@ struct Exec {
   // buffer ([N, O], or [parts, N, O] float32 with *parts >= 2).
   void* linear(const void* x, const Matrix& m, int n, bool out_f32, bool partial_ok, bool use_packed, int* parts, long ldx = 0);
   void linear_into(const void* x, const Matrix& m, int n, bool out_f32, bool use_packed, void* y);
+  // takes a delta's open sum: two float32 partial sums
+  void plain(Pending& d);
   // adds what is pending and makes sure the bfloat16 mirror of x exists
   void with_mirror(float* x, Pending& pending, void** mirror);
   // adds what is pending into x
@@ -354,10 +364,12 @@ struct Plan {
   int own_gemm = 0;         // products above the few-row kernels' range: 0 the library's, 1 the tiled kernel
   std::vector<std::unique_ptr<NormPart>> norms;
   std::vector<std::unique_ptr<Body>> bodies;
-  enum { OP_HALF, OP_NORM, OP_BODY, OP_ADD, OP_DROP, OP_NORM_DELTA, OP_REINJECT, OP_ADD_NORMED, OP_STREAMS_NORM, OP_STREAMS_ADD, OP_ROWS };
+  enum { OP_HALF, OP_NORM, OP_BODY, OP_ADD, OP_DROP, OP_NORM_DELTA, OP_REINJECT, OP_ADD_NORMED, OP_STREAMS_NORM, OP_STREAMS_ADD, OP_ROWS, OP_SUM };
   struct Op {
     int kind, norm, body, value;   // value: what a body reads, an add adds, a drop drops
     int result;                    // the value that a norm or a body makes
+    int value2 = -1;               // a sum's second value, and what the two are multiplied by
+    float scale = 1.f, scale2 = 1.f;
   };
   std::vector<Op> ops;
   int n_values = 0;
@@ -396,6 +408,14 @@ void Exec::with_mirror(float* x, Pending& pending, void** mirror) {
                                 std::max(pending.parts, 1), count, *mirror, count, a.stream));
   give(pending.data);
   pending = Pending{};
+}
+void Exec::plain(Pending& d) {
+  if (d.parts == 0 || d.is_plain()) return;
+  Pending out{take(2L * a.n_rows * p.hidden * 4), 2};
+  RUN(*this, gibbs_rows_terms(d.data, d.parts, d.bias, d.scale, d.data2, std::max(d.parts2, 1), d.scale2, (float*)out.data, p.dtype, a.n_rows, p.hidden, a.stream));
+  give(d.data);
+  give(d.data2);
+  d = out;
 }
 void Exec::settle(float* x, Pending& pending) {
   if (pending.parts == 0) return;
@@ -693,6 +713,10 @@ struct AttnBody : Body {
   int chunk = 0;
   float softcap = 0.f;
   int gate_off = -1;                  // where the gate's columns start in a projected row (< 0: no gate)
+  // what gibbs_plan_attention_whole_norm sets: q and k normed over the whole projection (gains in the stored layout), and a mixer that
+  // reads another's pages may have the projection options; and gibbs_plan_attention_out_bias: a bias on the result
+  bool whole_norm = false;
+  const float* out_bias = nullptr;
   bool extras() const { return !general_prep && (vd != hd || unit_qk || temp_every > 0 || bias); }
   int cache_group() const override { return group; }
   // the fast kernels know rotations only (or no encoding at all)
@@ -733,6 +757,12 @@ struct AttnBody : Body {
     const int* table = e.table(group);
     const int width = e.width(group);
     if (general_prep) {
+      if (whole_norm) {
+        RUN(e, gibbs_qkv_prepare_whole(raw, ldq, owns ? kpages : nullptr, owns ? vpages : nullptr, e.p.dtype, prep_q_gain, prep_k_gain, prep_eps, prep_norm_dim,
+                                       inv_freq, rot, variant, cos_sin, table_len, e.a.pos, e.a.row_req, table, width, page_size, num_pages, N, nh, kv, hd, vd,
+                                       e.a.stream));
+        return;
+      }
       // bias, rotation, value mixing and the cache write in one pass; the values that later layers mix into theirs
       // stay in a buffer of the step
       void* keep = nullptr;
@@ -803,6 +833,7 @@ struct AttnBody : Body {
     e.give(raw);
     Pending delta;
     delta.data = e.linear(att, out, N, false, true, true, &delta.parts);
+    delta.bias = out_bias;
     e.give(att);
     return delta;
   }
@@ -1183,6 +1214,119 @@ struct GatedOuterBody : Body {
   }
 };
 
+// ---- gated linear attention
+// One product gives [q | k | v | g | the gate's low-rank columns] of the rows (segments start at multiples of 8 values); the rule, the
+// heads' norm and the output gate are one kernel for decoded tokens and short portions, three for long ones (gated_linear.hip).
+struct GatedLinearBody : Body {
+  Matrix in, out, z2;                // z2 [H D, rank]: the second matrix of the gate's pair
+  int H = 0, D = 0, V = 0, rank = 0, off_q = 0, off_k = 0, off_v = 0, off_g = 0, off_z = 0;
+  const float* bias = nullptr;       // [H D]
+  const float* gain = nullptr;       // [V]
+  float* rule_state = nullptr;       // [slots][H][D][V]
+  long slot_stride = 0;
+  float eps = 0.f, inv_tau = 1.f, q_scale = 1.f;
+  Pending general(Exec& e, void* h) const override {
+    const GibbsStepArgs& a = e.a;
+    const int N = a.n_rows;
+    char* raw = (char*)e.linear(h, in, N, false, false, true, nullptr);
+    void* y = e.take((long)N * H * V * e.esize);
+    // (requests at the head of the batch that bring one row each: row n is request n's)
+    const int lead = e.rows_are_requests() ? N : a.lead_single;
+    const int rest = N - lead, reqs = a.n_req - lead;
+    auto walk = [&](const int* cu, const int* slot, int n) {
+      RUN(e, gibbs_gated_linear_rows(raw, in.O, off_q, off_k, off_v, off_g, off_z, z2.w, rank, bias, inv_tau, q_scale, gain, eps, rule_state, slot_stride, cu, slot,
+                                     y, e.p.dtype, n, H, D, V, a.stream));
+    };
+    if (lead > 0) walk(nullptr, a.slot, lead);
+    if (rest > 0 && a.max_q >= WALKED_ROWS && gibbs_gated_linear_chunks_take(D, V)) {
+      float* z = (float*)e.linear(raw + ((long)lead * in.O + off_z) * e.esize, z2, rest, true, false, false, nullptr, in.O);
+      float* work = (float*)e.take(gibbs_gated_linear_chunks_workspace(rest, reqs, H, D, V) * 4);
+      RUN(e, gibbs_gated_linear_chunks(raw, in.O, off_q, off_k, off_v, off_g, z, bias, inv_tau, q_scale, gain, eps, rule_state, slot_stride, a.cu + lead,
+                                       a.slot + lead, y, work, e.p.dtype, rest, reqs, H, D, V, a.stream));
+      e.give(work);
+      e.give(z);
+    } else if (rest > 0) {
+      walk(a.cu + lead, a.slot + lead, reqs);
+    }
+    e.give(raw);
+    Pending delta;
+    delta.data = e.linear(y, out, N, false, true, true, &delta.parts);
+    e.give(y);
+    return delta;
+  }
+};
+
+// ---- matrix memory with exponential gates and a normaliser
+// One product gives [q | k | v | g] of the rows; the two gates per head are float32 products of the rows by themselves: inside the row
+// kernel for decoded tokens and short portions, for long ones as w_gates h' (few "rows" of w_gates over the step's rows as the matrix:
+// the few-row product, which leaves every head's gates side by side along the tokens).
+struct MatrixLstmBody : Body {
+  Matrix in, out;
+  const void* w_gates = nullptr;     // [2 H, hidden]
+  const float* b_gates = nullptr;    // [2 H]
+  const float* gain = nullptr;       // [H V]
+  float* rule_state = nullptr;       // [slots][H][D][V]
+  float* norm_state = nullptr;       // [slots]([H][D], [H])
+  long slot_stride = 0;
+  int H = 0, D = 0, V = 0, off_q = 0, off_k = 0, off_v = 0, off_g = 0;
+  float eps = 0.f, cap = 1.f, q_scale = 1.f;
+  Pending general(Exec& e, void* h) const override {
+    const GibbsStepArgs& a = e.a;
+    const int N = a.n_rows, W = e.p.hidden;
+    void* raw = e.linear(h, in, N, false, false, true, nullptr);
+    void* y = e.take((long)N * H * V * e.esize);
+    const int lead = e.rows_are_requests() ? N : a.lead_single;
+    const int rest = N - lead, reqs = a.n_req - lead;
+    auto walk = [&](const int* cu, const int* slot, int n) {
+      RUN(e, gibbs_matrix_lstm_rows(raw, in.O, off_q, off_k, off_v, off_g, h, W, w_gates, b_gates, gain, cap, eps, q_scale, rule_state, norm_state, slot_stride, cu,
+                                    slot, y, e.p.dtype, n, H, D, V, a.stream));
+    };
+    if (lead > 0) walk(nullptr, a.slot, lead);
+    if (rest > 0 && a.max_q >= WALKED_ROWS && gibbs_matrix_lstm_chunks_take(D, V)) {
+      const Matrix rows{(char*)h + (long)lead * W * e.esize, nullptr, rest, W};
+      float* gates = (float*)e.linear(w_gates, rows, 2 * H, true, false, false, nullptr);
+      float* work = (float*)e.take(gibbs_matrix_lstm_chunks_workspace(rest, reqs, H, D, V) * 4);
+      RUN(e, gibbs_matrix_lstm_chunks(raw, in.O, off_q, off_k, off_v, off_g, h, W, w_gates, b_gates, gain, cap, eps, q_scale, rule_state, norm_state, slot_stride,
+                                      a.cu + lead, a.slot + lead, y, gates, work, e.p.dtype, rest, reqs, H, D, V, a.stream));
+      e.give(work);
+      e.give(gates);
+    } else if (rest > 0) {
+      walk(a.cu + lead, a.slot + lead, reqs);
+    }
+    e.give(raw);
+    Pending delta;
+    delta.data = e.linear(y, out, N, false, true, true, &delta.parts);
+    e.give(y);
+    return delta;
+  }
+};
+
+// ---- dense feed-forward without a gate: down(act(up h)), optionally times the entries of the row's token in a second table in between
+struct ActMlpBody : Body {
+  Matrix up, down;                    // down's inner size may be wider than F, with columns of zeros
+  int F = 0, act = 0;
+  const void* mult = nullptr;         // [vocab, mult_ld] in the run's compute type, or null
+  long mult_ld = 0;
+  int vocab = 0;
+  Pending general(Exec& e, void* h) const override {
+    const GibbsStepArgs& a = e.a;
+    const int N = a.n_rows, Fs = down.I;
+    if (mult && !a.ids && !e.status) e.status = gibbs_fail("step: a feed-forward that reads the rows' tokens needs them");
+    void* y = e.take((long)N * Fs * e.esize);
+    if (e.few_rows && Fs == F && up.I % 8 == 0) {
+      RUN(e, gibbs_skinny_act(h, up.packed ? up.packed : up.w, y, N, F, up.I, up.I, up.packed ? 0 : up.I, Fs, act, mult, mult_ld, a.ids, vocab, a.stream));
+    } else {
+      void* z = e.linear(h, up, N, false, false, true, nullptr);
+      RUN(e, gibbs_act_rows(z, y, Fs, e.p.dtype, act, mult, mult_ld, a.ids, vocab, N, F, a.stream));
+      e.give(z);
+    }
+    Pending delta;
+    delta.data = e.linear(y, down, N, false, true, true, &delta.parts);
+    e.give(y);
+    return delta;
+  }
+};
+
 // ---- dense feed-forward without a gate: down(act(up h)), act a polynomial of row-normed powers
 struct MlpBody : Body {
   Matrix up, down;
@@ -1221,6 +1365,7 @@ struct MoeBody : Body {
   // their sum; the router's last `identity` outputs are experts without matrices whose result is the row itself
   // mode 2: scores by the sigmoid of every output alone, weights the chosen scores as they are
   int mode = 0, identity = 0;
+  float weight_scale = 1.f;   // mode 1: the weights times a constant
   bool weigh_input = false;   // the weight multiplies the expert's input (its gate and up products) instead of its result
   Pending general(Exec& e, void* h) const override {
     const int N = e.a.n_rows, W = e.p.hidden, pairs = N * top;
@@ -1229,7 +1374,7 @@ struct MoeBody : Body {
     int* chosen = (int*)e.take((long)pairs * 4);
     float* weight = (float*)e.take((long)pairs * 4);
     float* sgate = shared_gate ? (float*)e.take((long)N * 4) : nullptr;
-    RUN(e, gibbs_moe_route_mode(h, W, e.p.dtype, router, router_bias, shared_gate, chosen, weight, sgate, N, W, E + identity, top, mode, e.a.stream));
+    RUN(e, gibbs_moe_route_scaled(h, W, e.p.dtype, router, router_bias, shared_gate, chosen, weight, sgate, N, W, E + identity, top, mode, weight_scale, e.a.stream));
     int* sorted = (int*)e.take(cap * 4);
     int* place = (int*)e.take((long)pairs * 4);
     int* tile_expert = (int*)e.take(cap / bm * 4);
@@ -1342,6 +1487,7 @@ void Exec::run() {
         } else {
           void* h = n.run(*this, x, pending, nullptr, N);
           pending = b.general(*this, h);
+          plain(pending);
           give(h);
           give(mirror);
           mirror = nullptr;
@@ -1359,16 +1505,29 @@ void Exec::run() {
       case Plan::OP_ROWS: {
         // a body whose result is read as rows by the next body (a filter on what a mixer reads), not added to the stream
         Pending made = p.bodies[op.body]->general(*this, rows[op.value]);
+        plain(made);
         if (made.parts != 1 && !status) status = gibbs_fail("step: a body whose result is read as rows must give whole rows");
         rows[op.result] = made.data;
         break;
       }
       case Plan::OP_ADD:
         settle(x, pending);
+        plain(deltas[op.value]);
         pending = deltas[op.value];
         deltas[op.value] = Pending{};
         break;
+      case Plan::OP_SUM: {
+        Pending &one = deltas[op.value], &two = deltas[op.value2];
+        if (one.data2) plain(one);
+        if (two.bias || two.data2 || two.scale != 1.f) plain(two);
+        Pending sum{one.data, one.parts, one.bias, one.scale * op.scale, two.data, two.parts, op.scale2};
+        one = Pending{};
+        two = Pending{};
+        deltas[op.result] = sum;
+        break;
+      }
       case Plan::OP_NORM_DELTA:
+        plain(deltas[op.value]);
         deltas[op.result] = p.norms[op.norm]->run_on(*this, deltas[op.value]);
         deltas[op.value] = Pending{};
         break;
@@ -1391,7 +1550,17 @@ void Exec::run() {
           void* out = with_rows ? take((long)N * H * esize) : nullptr;
           int fused = -1;
           const bool mixed = deferred.delta && deferred.delta == d.data;
-          if (!dry && status == 0) {
+          const bool summed = !d.is_plain();
+          if (summed && reader == 2) {
+            // (the shifted reader runs behind the pass that sums)
+            give(out);
+            out = nullptr;
+          }
+          if (!dry && status == 0 && summed) {
+            fused = gibbs_rmsnorm_rows_sum_add_read(x, d.data, std::max(d.parts, 1), (long)N * H, d.bias, d.scale, d.data2, std::max(d.parts2, 1), d.scale2, gain_d,
+                                                    eps_d, reader == 1 && with_rows ? 1 : 0, out, p.dtype, N, H, a.stream);
+            if (fused > 0) status = 1;
+          } else if (!dry && status == 0) {
             fused = gibbs_rmsnorm_rows_add_read(x, mixed ? deferred.y : d.data, mixed ? 1 : std::max(d.parts, 1), (long)N * H, mixed ? deferred.place : nullptr,
                                                 mixed ? deferred.weight : nullptr, mixed ? deferred.top : 0, mixed ? deferred.shared : nullptr,
                                                 mixed ? deferred.gate : nullptr, gain_d, eps_d, reader, mu, shift_state, shift_stride, a.slot, out, p.dtype, N, H,
@@ -1403,10 +1572,11 @@ void Exec::run() {
           if (fused == 0) {
             if (mixed) mix_done();
             give(d.data);
+            give(d.data2);
             d = Pending{};
             give(mirror);
             mirror = nullptr;
-            if (with_rows) {
+            if (out) {
               rows[next->result] = out;
               ++i;
             }
@@ -1414,6 +1584,24 @@ void Exec::run() {
           }
           give(out);
         }
+        if (!d.is_plain() && !next && pending.parts == 0 && p.norms[op.norm]->plain_rms(&gain_d, &eps_d)) {
+          // (the last sublayer's boundary: nothing is read behind it)
+          int fused = dry && H % 4 == 0 && H <= 16384 ? 0 : -1;
+          if (!dry && status == 0) {
+            fused = gibbs_rmsnorm_rows_sum_add_read(x, d.data, std::max(d.parts, 1), (long)N * H, d.bias, d.scale, d.data2, std::max(d.parts2, 1), d.scale2, gain_d,
+                                                    eps_d, 0, nullptr, p.dtype, N, H, a.stream);
+            if (fused > 0) status = 1;
+          }
+          if (fused == 0) {
+            give(d.data);
+            give(d.data2);
+            d = Pending{};
+            give(mirror);
+            mirror = nullptr;
+            break;
+          }
+        }
+        plain(d);
         if (next && pending.parts == 0 && d.data && p.norms[op.norm]->plain_rms(&gain_d, &eps_d) && p.norms[next->norm]->plain_rms(&gain_n, &eps_n)) {
           void* out = take((long)N * H * esize);
           int fused = -1;
@@ -1484,6 +1672,7 @@ void Exec::run() {
         // same pass (the rows are in registers already: a sublayer's boundary is one kernel, not two)
         const Hyper& hc = p.hypers[op.body];
         Pending& d = deltas[op.value];
+        plain(d);
         const Plan::Op* next = i + 1 < last && p.ops[i + 1].kind == Plan::OP_STREAMS_NORM ? &p.ops[i + 1] : nullptr;
         int kind = 0;
         const float *gain = nullptr, *bias = nullptr;
@@ -1504,6 +1693,7 @@ void Exec::run() {
       case Plan::OP_DROP:
         give(rows[op.value]);
         give(deltas[op.value].data);
+        give(deltas[op.value].data2);
         rows[op.value] = nullptr;
         deltas[op.value] = Pending{};
         break;
@@ -1521,7 +1711,7 @@ void Exec::run() {
   if (a.settle) settle(x, pending);
   give(pending.data);
   for (void* r : rows) give(r);
-  for (Pending& d : deltas) give(d.data);
+  for (Pending& d : deltas) { give(d.data); give(d.data2); }
   give(mirror);      // (buffers of the caller's are not the arena's: giving them back does nothing)
   for (auto& kv : published) give(kv.second);
   published.clear();
@@ -1746,6 +1936,63 @@ GIBBS_EXPORT int gibbs_plan_body_gated_outer(void* plan, const GibbsGatedOuterSp
   return (int)p->bodies.size() - 1;
 }
 
+GIBBS_EXPORT int gibbs_plan_body_gated_linear(void* plan, const GibbsGatedLinearSpec* d) {
+  Plan* p = open_plan(plan);
+  if (!p) return -1;
+  if (!d || !(d->w_in && d->w_out && d->w_z && d->z_bias && d->gain && d->rule_state && d->heads > 0 && d->heads <= 65535 && d->dim > 0 && d->vdim > 0 && d->rank > 0 &&
+              d->tau > 0.f && d->slot_stride >= (long)d->heads * d->dim * d->vdim && gibbs_gated_linear_rows_take(d->dim, d->vdim))) {
+    gibbs_fail("plan: bad gated linear attention");
+    return -1;
+  }
+  auto b = std::make_unique<GatedLinearBody>();
+  b->in = Matrix{d->w_in, d->p_in, d->in_rows, p->hidden};
+  b->out = Matrix{d->w_out, d->p_out, p->hidden, d->heads * d->vdim};
+  b->z2 = Matrix{d->w_z, nullptr, d->heads * d->dim, d->rank};
+  b->H = d->heads; b->D = d->dim; b->V = d->vdim; b->rank = d->rank;
+  b->off_q = d->off_q; b->off_k = d->off_k; b->off_v = d->off_v; b->off_g = d->off_g; b->off_z = d->off_z;
+  b->bias = d->z_bias; b->gain = d->gain; b->rule_state = d->rule_state; b->slot_stride = d->slot_stride;
+  b->eps = d->eps; b->inv_tau = 1.0f / d->tau; b->q_scale = d->q_scale;
+  p->bodies.push_back(std::move(b));
+  return (int)p->bodies.size() - 1;
+}
+
+GIBBS_EXPORT int gibbs_plan_body_matrix_lstm(void* plan, const GibbsMatrixLstmSpec* d) {
+  Plan* p = open_plan(plan);
+  if (!p) return -1;
+  if (!d || !(d->w_in && d->w_out && d->w_gates && d->b_gates && d->gain && d->rule_state && d->norm_state && d->heads > 0 && d->heads <= 65535 && d->dim > 0 &&
+              d->vdim > 0 && d->cap > 0.f && d->slot_stride >= (long)d->heads * d->dim * d->vdim && d->slot_stride >= (long)d->heads * (d->dim + 1) &&
+              gibbs_matrix_lstm_rows_take(d->dim, d->vdim))) {
+    gibbs_fail("plan: bad matrix memory");
+    return -1;
+  }
+  auto b = std::make_unique<MatrixLstmBody>();
+  b->in = Matrix{d->w_in, d->p_in, d->in_rows, p->hidden};
+  b->out = Matrix{d->w_out, d->p_out, p->hidden, d->heads * d->vdim};
+  b->w_gates = d->w_gates; b->b_gates = d->b_gates; b->gain = d->gain;
+  b->rule_state = d->rule_state; b->norm_state = d->norm_state; b->slot_stride = d->slot_stride;
+  b->H = d->heads; b->D = d->dim; b->V = d->vdim;
+  b->off_q = d->off_q; b->off_k = d->off_k; b->off_v = d->off_v; b->off_g = d->off_g;
+  b->eps = d->eps; b->cap = d->cap; b->q_scale = d->q_scale;
+  p->bodies.push_back(std::move(b));
+  return (int)p->bodies.size() - 1;
+}
+
+GIBBS_EXPORT int gibbs_plan_body_act_mlp(void* plan, const void* w_up, const void* p_up, const void* w_down, const void* p_down, int F, int F_stored, int act,
+                                         const void* mult, long mult_ld, int vocab) {
+  Plan* p = open_plan(plan);
+  if (!p) return -1;
+  if (!(w_up && w_down && F > 0 && F_stored >= F && ((act >= 0 && act < 4) || act == 5) && (!mult || (mult_ld >= F && vocab > 0)))) {
+    gibbs_fail("plan: bad feed-forward without a gate: width %d (stored %d), activation %d", F, F_stored, act);
+    return -1;
+  }
+  auto b = std::make_unique<ActMlpBody>();
+  b->up = Matrix{w_up, p_up, F, p->hidden};
+  b->down = Matrix{w_down, p_down, p->hidden, F_stored};
+  b->F = F; b->act = act; b->mult = mult; b->mult_ld = mult_ld; b->vocab = vocab;
+  p->bodies.push_back(std::move(b));
+  return (int)p->bodies.size() - 1;
+}
+
 GIBBS_EXPORT int gibbs_plan_embedding_norm(void* plan, const float* gain, float eps) {
   Plan* p = open_plan(plan);
   if (!p) return -1;
@@ -1837,15 +2084,35 @@ GIBBS_EXPORT int gibbs_plan_attention_projection(void* plan, int body, int vd, c
   if (!p) return -1;
   AttnBody* t = p->has_body(body) ? dynamic_cast<AttnBody*>(p->bodies[body].get()) : nullptr;
   if (!t || vd <= 0 || keep_mode < 0 || keep_mode > 2) { gibbs_fail("plan: body %d is no attention, or bad projection options", body); return -1; }
-  if (t->q_gain || t->k_gain || t->hook || t->unit_qk || t->temp_every > 0 || !t->owns) {
-    gibbs_fail("plan: an attention with projection biases, a sink or value mixing has no q/k norm, no hook and no temperature, and owns its pages");
+  if (t->q_gain || t->k_gain || t->hook || t->unit_qk || t->temp_every > 0 || (!t->owns && (bias || keep_mode))) {
+    gibbs_fail("plan: an attention with projection biases, a sink or value mixing has no q/k norm, no hook and no temperature, and owns its pages (a sink alone: or reads another's)");
     return -1;
   }
   if (keep_mode && !(vt > 0 && vt <= vd && keep_key >= 0 && (keep_mode == 1 || lambda))) { gibbs_fail("plan: value mixing needs a key, the values' size and its weight"); return -1; }
   t->general_prep = true;
   t->vd = vd; t->proj_bias = bias; t->sink = sink; t->keep_mode = keep_mode; t->keep_key = keep_key; t->vt = vt; t->lambda = lambda;
-  t->qkv.O = (t->nh + t->nkv) * t->hd + t->nkv * vd;
+  t->qkv.O = t->owns ? (t->nh + t->nkv) * t->hd + t->nkv * vd : t->nh * t->hd;
   t->out.I = t->nh * vd;
+  return 0;
+}
+GIBBS_EXPORT int gibbs_plan_attention_whole_norm(void* plan, int body, const float* q_gain, const float* k_gain, float eps, int norm_dim) {
+  Plan* p = open_plan(plan);
+  if (!p) return -1;
+  AttnBody* t = p->has_body(body) ? dynamic_cast<AttnBody*>(p->bodies[body].get()) : nullptr;
+  if (!t || !t->general_prep || t->proj_bias || t->keep_mode || t->v_from_k || t->v_inv_freq || t->prep_q_gain || !q_gain || (t->owns && !k_gain) || norm_dim <= 0 || norm_dim > t->hd) {
+    gibbs_fail("plan: body %d is no attention with projection options that a norm over the whole projection goes with", body);
+    return -1;
+  }
+  t->whole_norm = true;
+  t->prep_q_gain = q_gain; t->prep_k_gain = k_gain; t->prep_eps = eps; t->prep_norm_dim = norm_dim;
+  return 0;
+}
+GIBBS_EXPORT int gibbs_plan_attention_out_bias(void* plan, int body, const float* bias) {
+  Plan* p = open_plan(plan);
+  if (!p) return -1;
+  AttnBody* t = p->has_body(body) ? dynamic_cast<AttnBody*>(p->bodies[body].get()) : nullptr;
+  if (!t || !t->general_prep || !bias) { gibbs_fail("plan: body %d is no attention with projection options, or no bias on its result", body); return -1; }
+  t->out_bias = bias;
   return 0;
 }
 
@@ -1927,6 +2194,15 @@ GIBBS_EXPORT int gibbs_plan_moe_scores(void* plan, int body, int mode, int ident
   MoeBody* m = p->has_body(body) ? dynamic_cast<MoeBody*>(p->bodies[body].get()) : nullptr;
   if (!m || mode < 0 || mode > 2 || identity < 0 || m->E + identity > 1024 || m->top > m->E + identity) { gibbs_fail("plan: body %d is no mixture of experts, or bad router options", body); return -1; }
   m->mode = mode; m->identity = identity;
+  return 0;
+}
+
+GIBBS_EXPORT int gibbs_plan_moe_weight_scale(void* plan, int body, float scale) {
+  Plan* p = open_plan(plan);
+  if (!p) return -1;
+  MoeBody* m = p->has_body(body) ? dynamic_cast<MoeBody*>(p->bodies[body].get()) : nullptr;
+  if (!m || m->mode != 1) { gibbs_fail("plan: body %d is no mixture of experts whose scores are a softmax over all outputs", body); return -1; }
+  m->weight_scale = scale;
   return 0;
 }
 
@@ -2060,6 +2336,14 @@ GIBBS_EXPORT int gibbs_plan_op_add(void* plan, int value) {
   if (!known_value(p, value)) { gibbs_fail("plan: no value %d to add", value); return -1; }
   return append(p, Plan::OP_ADD, -1, -1, value, false);
 }
+GIBBS_EXPORT int gibbs_plan_op_sum(void* plan, int value, float scale, int value2, float scale2) {
+  Plan* p = open_plan(plan);
+  if (!p) return -1;
+  if (!known_value(p, value) || !known_value(p, value2) || value == value2) { gibbs_fail("plan: no values %d and %d to sum", value, value2); return -1; }
+  const int made = append(p, Plan::OP_SUM, -1, -1, value, true);
+  p->ops.back().value2 = value2; p->ops.back().scale = scale; p->ops.back().scale2 = scale2;
+  return made;
+}
 GIBBS_EXPORT int gibbs_plan_op_drop(void* plan, int value) {
   Plan* p = open_plan(plan);
   if (!p) return -1;
@@ -2137,6 +2421,7 @@ GIBBS_EXPORT long gibbs_plan_body_forward(const void* plan, int body, const Gibb
   Exec e(*p, *args);
   Pending delta = p->bodies[body]->general(e, (void*)h);
   e.mix_now();
+  e.plain(delta);
   if (e.status) return -1;
   if (e.dry) return e.arena.peak;
   *out_offset = (char*)delta.data - (char*)args->workspace;

@@ -184,6 +184,43 @@ struct GibbsGatedOuterSpec {
   float eps;
 };
 int gibbs_plan_body_gated_outer(void* plan, const struct GibbsGatedOuterSpec* spec);
+// Gated linear attention: w_in [in_rows, hidden], rows with q and k (heads * dim) at off_q, off_k, v and the output gate (heads * vdim) at
+// off_v, off_g, and the first matrix of the decay's low-rank pair (rank) at off_z; w_z [heads * dim, rank] the second, z_bias [heads *
+// dim]; per head f = sigmoid(z + z_bias)^(1 / tau), S = diag(f) S + k v', read-out S' (q_scale q) divided by its root mean square, times
+// gain [vdim], times silu of the gate.  p_in, p_out: w_in and w_out in tile order, or null.  rule_state [slots][heads][dim][vdim].
+struct GibbsGatedLinearSpec {
+  const void* w_in; const void* p_in; const void* w_out; const void* p_out; const void* w_z;
+  const float* z_bias; const float* gain;
+  float* rule_state; long slot_stride;
+  int in_rows, heads, dim, vdim, rank, off_q, off_k, off_v, off_g, off_z;
+  float eps, tau, q_scale;
+};
+int gibbs_plan_body_gated_linear(void* plan, const struct GibbsGatedLinearSpec* spec);
+// Matrix memory with exponential gates: w_in [in_rows, hidden], rows with q and k (heads * dim), v and the output gate (heads * vdim) at
+// their offsets; w_gates [2 heads, hidden] and b_gates [2 heads]: the logarithms of the input gates and, before log sigmoid, of the
+// forget gates, both capped as cap tanh(. / cap); S, n and m as in matrix_lstm.hip, read-out divided by its root mean square, times gain
+// [heads * vdim], times sigmoid of the output gate.  rule_state [slots][heads][dim][vdim], norm_state [slots]([heads][dim], [heads]).
+struct GibbsMatrixLstmSpec {
+  const void* w_in; const void* p_in; const void* w_out; const void* p_out; const void* w_gates;
+  const float* b_gates; const float* gain;
+  float* rule_state; float* norm_state; long slot_stride;
+  int in_rows, heads, dim, vdim, off_q, off_k, off_v, off_g;
+  float eps, cap, q_scale;
+};
+int gibbs_plan_body_matrix_lstm(void* plan, const struct GibbsMatrixLstmSpec* spec);
+// Dense feed-forward without a gate: down(act(up h)), act a code of activation.h without a gate (0 .. 3, or 5: the square of relu).
+// mult (or null) [vocab, mult_ld] in the compute type: act(up h) is multiplied by the first F entries of the row's token there.  w_down
+// [hidden, F_stored] with columns of zeros from F on.
+int gibbs_plan_body_act_mlp(void* plan, const void* w_up, const void* p_up, const void* w_down, const void* p_down, int F, int F_stored, int act,
+                            const void* mult, long mult_ld, int vocab);
+// An attention body that takes the projection options (without biases on q, k, v): q and k divided by the root mean square of their whole
+// projections (over heads * norm_dim channels) and multiplied by gains in the stored layout ([heads * head size]; k_gain null for a
+// mixer that reads another's pages), before the rotation.
+int gibbs_plan_attention_whole_norm(void* plan, int body, const float* q_gain, const float* k_gain, float eps, int norm_dim);
+// An attention body that takes the projection options: bias [hidden] on its result.
+int gibbs_plan_attention_out_bias(void* plan, int body, const float* bias);
+// A mixture of experts in mode 1: the chosen experts' weights times a constant.
+int gibbs_plan_moe_weight_scale(void* plan, int body, float scale);
 // Differential attention: w_in [in_rows, hidden], rows [q: heads x 2 maps x dim | k: kv_heads x 2 maps x dim | v: kv_heads x
 // vdim | at gate_off (< 0: none) one gate per head]; every map normed (q_gain, k_gain [dim], eps) and its first `rot` entries
 // turned; two softmax maps per head over the same values, a_1 - lam a_2 (lam: one float32 on the device) divided by its root
@@ -238,6 +275,7 @@ int gibbs_plan_op_norm(void* plan, int norm);                 // -> value: norm(
 int gibbs_plan_op_body(void* plan, int body, int value);      // -> value: body(normed rows)
 int gibbs_plan_op_rows(void* plan, int body, int value);      // -> value: body(normed rows), read as rows by a later body
 int gibbs_plan_op_add(void* plan, int value);                 // x += delta (lazily: it stays pending for the next norm)
+int gibbs_plan_op_sum(void* plan, int value, float scale, int value2, float scale2);   // -> value: scale a + scale2 b of two bodies' deltas, which are used up
 int gibbs_plan_op_drop(void* plan, int value);                // the value is not read again
 int gibbs_plan_op_norm_delta(void* plan, int norm, int value);   // -> value: norm(a body's delta), the stream untouched
 int gibbs_plan_op_add_normed(void* plan, int norm, int value);   // x += norm(a body's delta), in one pass where the norm can

@@ -10,6 +10,7 @@ from .lib import KernelError, call, dtype_code, library, ptr, require_cuda, stre
 
 ROPE_VARIANTS = {"half_split": 0, "interleaved": 1}
 ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "gelu": 2, "relu": 3}     # csrc/activation.h
+PLAIN_ACTIVATIONS = dict(ACTIVATIONS, relu_squared=5)              # of a feed-forward without a gate
 MOE_SCORES = {"softmax_top": 0, "softmax_all": 1, "sigmoid": 2}                  # a router's scores (csrc/moe.hip)
 
 

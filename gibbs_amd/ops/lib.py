@@ -100,6 +100,25 @@ _SIGNATURES = {
                                c_int, c_int, c_void_p],
     "gibbs_gated_outer_chunks": [c_void_p, c_long, c_int, c_void_p, c_void_p, c_void_p, c_float, c_void_p, c_long, c_void_p, c_void_p, c_void_p,
                                  c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
+    "gibbs_gated_linear_rows": [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_float, c_float, c_void_p,
+                                c_float, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
+    "gibbs_gated_linear_chunks": [c_void_p, c_long, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_float, c_float, c_void_p, c_float,
+                                  c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
+    "gibbs_matrix_lstm_rows": [c_void_p, c_long, c_int, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_float, c_float,
+                               c_float, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
+    "gibbs_matrix_lstm_chunks": [c_void_p, c_long, c_int, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_float, c_float,
+                                 c_float, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
+                                 c_int, c_int, c_int, c_void_p],
+    "gibbs_act_rows": [c_void_p, c_void_p, c_long, c_int, c_int, c_void_p, c_long, c_void_p, c_int, c_int, c_int, c_void_p],
+    "gibbs_skinny_act": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_long, c_long, c_long, c_int, c_void_p, c_long, c_void_p, c_int,
+                         c_void_p],
+    "gibbs_qkv_prepare_whole": [c_void_p, c_long, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_float, c_int, c_void_p, c_int, c_int,
+                                c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
+    "gibbs_rmsnorm_rows_sum_add_read": [c_void_p, c_void_p, c_int, c_long, c_void_p, c_float, c_void_p, c_int, c_float, c_void_p, c_float, c_int,
+                                        c_void_p, c_int, c_int, c_int, c_void_p],
+    "gibbs_rows_terms": [c_void_p, c_int, c_void_p, c_float, c_void_p, c_int, c_float, c_void_p, c_int, c_int, c_int, c_void_p],
+    "gibbs_moe_route_scaled": [c_void_p, c_long, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
+                               c_int, c_float, c_void_p],
     "gibbs_head_norm_gate": [c_void_p, c_void_p, c_int, c_void_p, c_long, c_void_p, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p],
     "gibbs_gated_outer_rule": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
                                c_void_p],
@@ -184,6 +203,12 @@ _VALUE_SIGNATURES = {
     "gibbs_gated_outer_chunks_take": ([c_int, c_int], c_int),
     "gibbs_gated_outer_step_takes": ([c_int, c_int], c_int),
     "gibbs_gated_outer_chunks_workspace": ([c_int, c_int, c_int, c_int, c_int], c_long),
+    "gibbs_gated_linear_rows_take": ([c_int, c_int], c_int),
+    "gibbs_gated_linear_chunks_take": ([c_int, c_int], c_int),
+    "gibbs_gated_linear_chunks_workspace": ([c_int, c_int, c_int, c_int, c_int], c_long),
+    "gibbs_matrix_lstm_rows_take": ([c_int, c_int], c_int),
+    "gibbs_matrix_lstm_chunks_take": ([c_int, c_int], c_int),
+    "gibbs_matrix_lstm_chunks_workspace": ([c_int, c_int, c_int, c_int, c_int], c_long),
     "gibbs_ssd_chunked_workspace": ([c_int, c_int, c_int, c_int], c_long),
 }
 

@@ -28,7 +28,10 @@ their channels, pair m by p * base^(-2m / v_head_dim) in the rotation's pairing,
 turned back by the query's position); `chunk: n` (a row sees the keys of its own stretch of n positions, counted from
 position 0, instead of a window); `softcap: c` (scores become c tanh(s / c) after the scale); `sink: "zero"` (a sink whose
 number is 0 and not learned: one added to the softmax's denominator); `gate` (tensor `gate_proj` [heads * v_head_dim,
-hidden]: the heads' outputs times sigmoid(W_g h), h the rows that the projections read, before the out-projection).
+hidden]: the heads' outputs times sigmoid(W_g h), h the rows that the projections read, before the out-projection);
+`qk_norm: "whole"` (tensors `q_norm` [heads * head_dim], `k_norm` [kv_heads * head_dim]: the root mean square is the whole
+projection's, over all heads of q at once and all heads of k at once; it goes with another layer's cache as well); and
+`out_bias` (tensor `o_bias` [hidden], a bias on the result).
 """
 from __future__ import annotations
 
@@ -58,6 +61,7 @@ class AttentionMixer(Mixer):
         self.v_head_dim = int(p.get("v_head_dim") or self.head_dim)
         self.q_temperature = p.get("q_temperature")
         self.has_bias, self.has_sink = bool(p.get("bias")), bool(p.get("sink"))
+        self.has_out_bias, self.whole_norm = bool(p.get("out_bias")), self.qk_norm == "whole"
         self.zero_sink = p.get("sink") == "zero"
         self.value_mix = p.get("value_mix")
         self.values_from_keys = bool(p.get("values_from_keys"))
@@ -76,13 +80,15 @@ class AttentionMixer(Mixer):
             raise ValueError("turned values have an even size and are not mixed")
         if self.value_mix is not None and (self.source is not None or int(self.value_mix["key"]) < 0):
             raise ValueError("value mixing needs a key >= 0 and a mixer that owns its pages")
+        if self.whole_norm and (self.has_bias or self.value_mix is not None or self.gated_options and not self.chunk and not self.softcap):
+            raise ValueError("a norm over the whole projection goes with neither projection biases nor value mixing, values from keys, turned values or a gate")
         if (self.has_bias or self.has_sink or self.value_mix is not None) and (self.qk_norm == "unit" or self.q_temperature is not None
-                                                                              or self.source is not None):
+                                                                              or (self.source is not None and not self.whole_norm)):
             raise ValueError("projection biases, a sink and value mixing go with neither a unit norm nor a temperature nor another layer's cache")
         if self.heads % self.kv_heads:
             raise ValueError(f"{self.heads} heads are not a multiple of {self.kv_heads} kv heads")
-        if self.qk_norm not in (None, "before", "unit"):
-            raise ValueError(f"qk_norm {self.qk_norm!r} is not implemented (None, 'before' or 'unit')")
+        if self.qk_norm not in (None, "before", "unit", "whole"):
+            raise ValueError(f"qk_norm {self.qk_norm!r} is not implemented (None, 'before', 'unit' or 'whole')")
         if self.window is not None and int(self.window) <= 0:
             raise ValueError(f"attention window {self.window} must be positive")
         self.position = build_position(spec.position, self.head_dim)
@@ -130,10 +136,13 @@ class AttentionMixer(Mixer):
         if self.gated:
             decls.append(TensorDecl(t["gate_proj"], (self.heads * vd, H)))
         decls.append(TensorDecl(t["out_proj"], (H, self.heads * vd)))
-        if self.qk_norm == "before":
-            decls.append(TensorDecl(t["q_norm"], (hd,), FLOAT32, init="gain"))
+        if self.qk_norm in ("before", "whole"):
+            q_size, k_size = (self.heads * hd, self.kv_heads * hd) if self.whole_norm else (hd, hd)
+            decls.append(TensorDecl(t["q_norm"], (q_size,), FLOAT32, init="gain"))
             if self.source is None:
-                decls.append(TensorDecl(t["k_norm"], (hd,), FLOAT32, init="gain"))
+                decls.append(TensorDecl(t["k_norm"], (k_size,), FLOAT32, init="gain"))
+        if self.has_out_bias:
+            decls.append(TensorDecl(t["o_bias"], (H,), FLOAT32, init="bias"))
         if self.has_bias:
             decls += [TensorDecl(t["q_bias"], (self.heads * hd,), FLOAT32, init="bias"),
                       TensorDecl(t["k_bias"], (self.kv_heads * hd,), FLOAT32, init="bias"),
@@ -150,7 +159,8 @@ class AttentionMixer(Mixer):
         """Options that take the preparation of the step's rows with biases, partial rotation and value mixing."""
         rotated_own_values = (self.v_head_dim != self.head_dim and self.qk_norm is None and self.q_temperature is None
                               and self.spec.position is not None and self.spec.position.kind == "rope")
-        return self.has_bias or self.has_sink or self.value_mix is not None or rotated_own_values or self.gated_options
+        return (self.has_bias or self.has_sink or self.value_mix is not None or rotated_own_values or self.gated_options or self.whole_norm
+                or self.has_out_bias)
 
     def bind(self, weights: WeightStore, rt: Runtime) -> None:
         self.rt = rt
@@ -162,7 +172,7 @@ class AttentionMixer(Mixer):
         # out-projection: products with them are exactly zero).
         self.padded_dim = None
         pad = -(-max(self.head_dim, self.v_head_dim) // 16) * 16
-        if (rt.act_dtype == torch.bfloat16 and self.source is None and (self.qk_norm == "unit" or self.projection_options())
+        if (rt.act_dtype == torch.bfloat16 and (self.source is None or self.whole_norm) and (self.qk_norm == "unit" or self.projection_options())
                 and pad <= 128 and (self.head_dim, self.v_head_dim) != (pad, pad)):
             self.padded_dim = pad
             wq = self._pad_heads(wq, self.heads, self.head_dim, pad, rows=True)
@@ -203,8 +213,14 @@ class AttentionMixer(Mixer):
             self.v_inv_freq = torch.from_numpy(rope_inv_freq(self.v_head_dim, float(self.value_rotation["theta"]))).to(rt.device)
         if self.value_mix is not None and not self.value_mix.get("publish"):
             self.mix_weight = weights[t["value_mix"]].reshape(1).contiguous()
-        self.q_gain = weights[t["q_norm"]] if self.qk_norm == "before" else None
-        self.k_gain = weights[t["k_norm"]] if self.qk_norm == "before" and self.source is None else None
+        gains = self.qk_norm in ("before", "whole")
+        self.q_gain = weights[t["q_norm"]] if gains else None
+        self.k_gain = weights[t["k_norm"]] if gains and self.source is None else None
+        if self.whole_norm and self.padded_dim:        # (in the layout of a projected row: zeros behind every head's channels)
+            def spread(g, heads):
+                return None if g is None else torch.nn.functional.pad(g.view(heads, self.head_dim), (0, self.padded_dim - self.head_dim)).reshape(-1).contiguous()
+            self.q_gain, self.k_gain = spread(self.q_gain, self.heads), spread(self.k_gain, self.kv_heads)
+        self.out_bias = weights[t["o_bias"]].contiguous() if self.has_out_bias else None
         self.rot, self.slopes, self.pos_hook, self.score_bias = None, None, False, None
         if self.position is not None:
             self.position.bind(weights, rt)
@@ -228,7 +244,7 @@ class AttentionMixer(Mixer):
         return [(self.heads * self.head_dim + kv + gate, self.hidden), (self.hidden, self.heads * self.v_head_dim)]
 
     def small_tensors(self):
-        own = [t for t in (self.q_gain, self.k_gain, self.slopes, self.proj_bias, self.sinks, self.mix_weight, self.v_inv_freq) if t is not None]   # (a score table is the position's)
+        own = [t for t in (self.q_gain, self.k_gain, self.slopes, self.proj_bias, self.sinks, self.mix_weight, self.v_inv_freq, self.out_bias) if t is not None]   # (a score table is the position's)
         return own + ([] if self.position is None else list(self.position.small_tensors()))
 
     def fold_input_gain(self, gain: torch.Tensor) -> None:
@@ -262,10 +278,17 @@ class AttentionMixer(Mixer):
             plan.attention_projection(body, v_head_dim=vd, bias=self.proj_bias, sink=self.sinks,
                                       keep_mode=0 if mix is None else (1 if mix.get("publish") else 2),
                                       keep_key=-1 if mix is None else int(mix["key"]), value_dim=self.v_head_dim, weight=self.mix_weight)
+            if self.source is not None and not self.whole_norm:
+                raise ValueError("an attention that reads another layer's cache takes these options with a norm over the whole projection only")
             if self.gated_options or self.qk_norm == "before":
-                plan.attention_gated(body, q_gain=self.q_gain, k_gain=self.k_gain, qk_eps=self.qk_norm_eps, norm_dim=self.head_dim,
+                gain_q, gain_k = (None, None) if self.whole_norm else (self.q_gain, self.k_gain)
+                plan.attention_gated(body, q_gain=gain_q, k_gain=gain_k, qk_eps=self.qk_norm_eps, norm_dim=self.head_dim,
                                      values_from_keys=self.values_from_keys, v_inv_freq=self.v_inv_freq, v_rot=self.v_head_dim,
                                      chunk=self.chunk, softcap=self.softcap, gate=self.gated)
+            if self.whole_norm:
+                plan.attention_whole_norm(body, q_gain=self.q_gain, k_gain=self.k_gain, eps=self.qk_norm_eps, norm_dim=self.head_dim)
+            if self.out_bias is not None:
+                plan.attention_out_bias(body, self.out_bias)
         return body
 
     def _emit_body(self, plan, cache, hook, head_dim: int) -> int:

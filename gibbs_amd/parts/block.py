@@ -155,34 +155,44 @@ class PostNormBlock(Block):
         x = x + norm1(mixer(x));   x = x + norm2(ffn(x))
 
     Roles: `mixer`, `norm1`, and optionally `ffn` with `norm2` (a layer without a feed-forward), and optionally `mixer_input`: a
-    part with state of its own (kind `token_shift`) that makes the rows the mixer reads from the stream.  Norms may carry a scale
-    per channel (`NormSpec.scale`).  The norm of a sublayer's result, its addition into the float32 stream and the rows that
+    part with state of its own (kind `token_shift`) that makes the rows the mixer reads from the stream.  Instead of `mixer` a pair of
+    mixers `left` and `right` may read the same rows: the mixer is then left_scale * left + right_scale * right (the layer spec's
+    `params`, each 1 by default), a sum that the border below takes on its way.  `side` with `side_norm` is a third sublayer of the same
+    form behind the feed-forward.  Norms may carry a scale per channel (`NormSpec.scale`).  The norm of a sublayer's result, its addition into the float32 stream and the rows that
     the next sublayer reads are one pass where the step's shape allows it (csrc/step_plan.hip)."""
 
     def __init__(self, spec, hidden, layer_index):
         super().__init__(spec, hidden, layer_index)
-        self.has_ffn = "ffn" in self.named
-        missing = [r for r in ["mixer", "norm1"] + (["norm2"] if self.has_ffn else []) if r not in self.named]
+        self.has_ffn, self.has_side, self.pair = "ffn" in self.named, "side" in self.named, "left" in self.named
+        want = (["left", "right"] if self.pair else ["mixer"]) + ["norm1"] + (["norm2"] if self.has_ffn else []) + (["side_norm"] if self.has_side else [])
+        missing = [r for r in want if r not in self.named]
         if missing:
             raise ValueError(f"layer {spec.name!r} lacks the parts {missing}")
 
     def bind(self, weights, rt: Runtime) -> None:
         super().bind(weights, rt)
         if rt.act_dtype == torch.bfloat16:       # (tile-ordered copies for the few-row products of decode steps)
-            self.mixer.pack_matrices()
-            if self.has_ffn:
-                self.ffn.pack_matrices()
+            for role in ("mixer", "left", "right", "ffn", "side"):
+                if role in self.named:
+                    self.named[role].pack_matrices()
 
     def emit(self, plan, caches) -> None:
         through = self.named.get("mixer_input")
         reader = plan.stream_rows() if through is None else through.emit(plan, caches["mixer_input"])
-        subs = [(reader, self.mixer.emit(plan, caches["mixer"]), self.norm1)]
+        roles = ["left", "right"] if self.pair else ["mixer"]
+        subs = [(reader, [self.named[r].emit(plan, caches[r]) for r in roles], self.norm1)]
         if self.has_ffn:
-            subs.append((plan.stream_rows(), self.ffn.emit(plan), self.norm2))
-        for reader, body, after in subs:
+            subs.append((plan.stream_rows(), [self.ffn.emit(plan)], self.norm2))
+        if self.has_side:
+            subs.append((plan.stream_rows(), [self.side.emit(plan)], self.side_norm))
+        for reader, bodies, after in subs:
             h = plan.normed(reader)
-            delta = plan.apply(body, h)
+            deltas = [plan.apply(body, h) for body in bodies]
             plan.drop(h)
+            delta = deltas[0]
+            if len(deltas) == 2:
+                scales = [float(self.spec.params.get(k, 1.0)) for k in ("left_scale", "right_scale")]
+                delta = plan.weighted_sum(deltas[0], scales[0], deltas[1], scales[1])
             plan.add_normed(after.emit(plan), delta)
 
 

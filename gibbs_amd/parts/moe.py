@@ -9,7 +9,8 @@ per row (`shared: {"inter": F, "activation": .., "gate": bool}`).
 `scores: "softmax_all"` is another router: scores s = softmax(z) over all router outputs, the `top` largest of
 s + correction (tensor `correction`, one number per output, seen by the choice alone), weights the chosen experts' s
 divided by their sum (+ 1e-20).  `identity: n`: the router has `experts + n` outputs, and the last n of them are experts
-without matrices whose result is the row itself.  `shared.gate: False` adds the shared expert as it is.
+without matrices whose result is the row itself.  `weight_scale` multiplies those weights.  `shared.gate: False` adds the shared
+expert as it is.
 
 `scores: "sigmoid"` is a third router: scores s = sigmoid(z), the `top` largest of s + correction (without a correction: the
 largest z), weights the chosen experts' s as they are.  `weigh: "input"` puts a choice's weight on the expert's input instead
@@ -43,6 +44,9 @@ class MoeFeedForward(FeedForward):
         self.outputs = self.experts + self.identity         # rows of the router
         if self.scores not in ops.MOE_SCORES or self.identity < 0:
             raise ValueError(f"router scores {self.scores!r} (one of {sorted(ops.MOE_SCORES)}) with {self.identity} identity experts")
+        self.weight_scale = float(p.get("weight_scale", 1.0))
+        if self.weight_scale != 1.0 and self.scores != "softmax_all":
+            raise ValueError(f"weights times {self.weight_scale} go with scores by a softmax over all outputs, not {self.scores!r}")
         self.weigh = p.get("weigh", "output")
         if self.weigh not in ("output", "input") or (self.weigh == "input" and (self.identity or p.get("shared"))):
             raise ValueError(f"weights on an expert's {self.weigh!r} ('output', or 'input' without identity or shared experts)")

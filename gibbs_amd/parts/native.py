@@ -75,6 +75,22 @@ class GatedOuterSpec(ctypes.Structure):
                 ("rule_state", c_void_p), ("slot_stride", c_long), ("heads", c_int), ("dim", c_int), ("vdim", c_int), ("eps", ctypes.c_float)]
 
 
+class GatedLinearSpec(ctypes.Structure):
+    """GibbsGatedLinearSpec of csrc/step_plan_api.h."""
+    _fields_ = [("w_in", c_void_p), ("p_in", c_void_p), ("w_out", c_void_p), ("p_out", c_void_p), ("w_z", c_void_p), ("z_bias", c_void_p),
+                ("gain", c_void_p), ("rule_state", c_void_p), ("slot_stride", c_long), ("in_rows", c_int), ("heads", c_int), ("dim", c_int),
+                ("vdim", c_int), ("rank", c_int), ("off_q", c_int), ("off_k", c_int), ("off_v", c_int), ("off_g", c_int), ("off_z", c_int),
+                ("eps", ctypes.c_float), ("tau", ctypes.c_float), ("q_scale", ctypes.c_float)]
+
+
+class MatrixLstmSpec(ctypes.Structure):
+    """GibbsMatrixLstmSpec of csrc/step_plan_api.h."""
+    _fields_ = [("w_in", c_void_p), ("p_in", c_void_p), ("w_out", c_void_p), ("p_out", c_void_p), ("w_gates", c_void_p), ("b_gates", c_void_p),
+                ("gain", c_void_p), ("rule_state", c_void_p), ("norm_state", c_void_p), ("slot_stride", c_long), ("in_rows", c_int), ("heads", c_int),
+                ("dim", c_int), ("vdim", c_int), ("off_q", c_int), ("off_k", c_int), ("off_v", c_int), ("off_g", c_int),
+                ("eps", ctypes.c_float), ("cap", ctypes.c_float), ("q_scale", ctypes.c_float)]
+
+
 class DiffAttentionSpec(ctypes.Structure):
     """GibbsDiffAttentionSpec of csrc/step_plan_api.h."""
     _fields_ = [("w_in", c_void_p), ("w_out", c_void_p), ("q_gain", c_void_p), ("k_gain", c_void_p), ("lam", c_void_p), ("inv_freq", c_void_p),
@@ -132,6 +148,13 @@ def declare(lib) -> None:
         "gibbs_plan_embedding_norm": ([P, P, F], I),
         "gibbs_plan_stream_rows": ([P], I),
         "gibbs_plan_shifted_rows": ([P, P, P, LG], I),
+        "gibbs_plan_body_gated_linear": ([P, POINTER(GatedLinearSpec)], I),
+        "gibbs_plan_body_matrix_lstm": ([P, POINTER(MatrixLstmSpec)], I),
+        "gibbs_plan_body_act_mlp": ([P, P, P, P, P, I, I, I, P, LG, I], I),
+        "gibbs_plan_attention_whole_norm": ([P, I, P, P, F, I], I),
+        "gibbs_plan_attention_out_bias": ([P, I, P], I),
+        "gibbs_plan_moe_weight_scale": ([P, I, F], I),
+        "gibbs_plan_op_sum": ([P, I, F, I, F], I),
         "gibbs_plan_body_gated_outer": ([P, POINTER(GatedOuterSpec)], I),
         "gibbs_plan_body_diff_attention": ([P, POINTER(DiffAttentionSpec)], I),
         "gibbs_plan_op_rows": ([P, I, I], I),
@@ -329,6 +352,15 @@ class NativePlan:
         self._made(L.library().gibbs_plan_attention_gated(self.handle, int(body), qg, kg, float(qk_eps), int(norm_dim), int(values_from_keys),
                                                           vf, int(v_rot), int(chunk or 0), float(softcap or 0.0), int(gate)))
 
+    def attention_whole_norm(self, body: int, *, q_gain, k_gain, eps: float, norm_dim: int) -> None:
+        """q and k normed over their whole projections (gains in the stored layout), before the rotation."""
+        q, k = self._held(q_gain, k_gain)
+        self._made(L.library().gibbs_plan_attention_whole_norm(self.handle, int(body), q, k, float(eps), int(norm_dim)))
+
+    def attention_out_bias(self, body: int, bias: torch.Tensor) -> None:
+        (b,) = self._held(bias)
+        self._made(L.library().gibbs_plan_attention_out_bias(self.handle, int(body), b))
+
     def conv_input(self, *, taps: torch.Tensor, kernel: int, state: torch.Tensor) -> int:
         """rows -> rows + conv(rows): taps float32 [hidden, kernel], state float32 [slots, kernel - 1, hidden] in the arena."""
         assert taps.dtype == torch.float32 and taps.is_contiguous() and state.dtype == torch.float32
@@ -376,6 +408,40 @@ class NativePlan:
         d.heads, d.dim, d.vdim, d.eps = m.heads, m.dim, m.vdim, m.norm_eps
         return self._made(L.library().gibbs_plan_body_gated_outer(self.handle, ctypes.byref(d)))
 
+    def gated_linear(self, m, *, rule_state: torch.Tensor) -> int:
+        """The gated linear attention `m` (parts/gated_linear.py) over its state [slots, heads, dim, vdim] in the arena."""
+        assert rule_state.dtype == torch.float32
+        d = GatedLinearSpec()
+        d.w_in, d.p_in, d.w_out, d.p_out, d.w_z, d.z_bias, d.gain = self._held(m.w_in, m.p_in, m.w_out, m.p_out, m.w_z, m.z_bias, m.gain)
+        d.rule_state, d.slot_stride = rule_state.data_ptr(), int(rule_state.stride(0))
+        self.keep.append(rule_state)
+        d.in_rows, d.heads, d.dim, d.vdim, d.rank = m.w_in.shape[0], m.heads, m.dim, m.vdim, m.rank
+        d.off_q, d.off_k, d.off_v, d.off_g, d.off_z = m.off_q, m.off_k, m.off_v, m.off_g, m.off_z
+        d.eps, d.tau, d.q_scale = m.norm_eps, m.tau, m.q_scale
+        return self._made(L.library().gibbs_plan_body_gated_linear(self.handle, ctypes.byref(d)))
+
+    def matrix_lstm(self, m, *, rule_state: torch.Tensor, norm_state: torch.Tensor) -> int:
+        """The matrix memory `m` (parts/matrix_lstm.py) over its states in the arena: [slots, heads, dim, vdim], and n with m behind it."""
+        assert rule_state.dtype == torch.float32 and norm_state.dtype == torch.float32 and rule_state.stride(0) == norm_state.stride(0)
+        d = MatrixLstmSpec()
+        d.w_in, d.p_in, d.w_out, d.p_out, d.w_gates, d.b_gates, d.gain = self._held(m.w_in, m.p_in, m.w_out, m.p_out, m.w_gates, m.b_gates, m.gain)
+        d.rule_state, d.norm_state, d.slot_stride = rule_state.data_ptr(), norm_state.data_ptr(), int(rule_state.stride(0))
+        self.keep += [rule_state, norm_state]
+        d.in_rows, d.heads, d.dim, d.vdim = m.w_in.shape[0], m.heads, m.dim, m.vdim
+        d.off_q, d.off_k, d.off_v, d.off_g = m.off_q, m.off_k, m.off_v, m.off_g
+        d.eps, d.cap, d.q_scale = m.norm_eps, m.gate_cap, m.q_scale
+        return self._made(L.library().gibbs_plan_body_matrix_lstm(self.handle, ctypes.byref(d)))
+
+    def act_mlp(self, *, w_up, p_up, w_down, p_down, inter: int, activation: int, table: Optional[torch.Tensor] = None, column: int = 0) -> int:
+        """down(act(up h)); with `table` [vocab, columns] in the run's type times the row's token's entries from `column` on in between."""
+        u, pu, dn, pd = self._held(w_up, p_up, w_down, p_down)
+        mult, ld, vocab = None, 0, 0
+        if table is not None:
+            assert table.is_contiguous() and table.dtype == self.rt.act_dtype and 0 <= column <= table.shape[1] - inter
+            self.keep.append(table)
+            mult, ld, vocab = table.data_ptr() + column * table.element_size(), int(table.shape[1]), int(table.shape[0])
+        return self._made(L.library().gibbs_plan_body_act_mlp(self.handle, u, pu, dn, pd, int(inter), int(w_down.shape[1]), int(activation), mult, ld, vocab))
+
     def differential_attention(self, m, *, kpages: torch.Tensor, vpages: torch.Tensor, group: int, stored) -> int:
         """The differential-attention mixer `m` (parts/diff_attention.py) over its pages [num_pages, kv_heads, page_size, size]."""
         from ..ops import ROPE_VARIANTS
@@ -414,6 +480,8 @@ class NativePlan:
         body = self._made(L.library().gibbs_plan_body_moe(self.handle, ctypes.byref(d)))
         if m.scores != "softmax_top" or m.identity:
             self._made(L.library().gibbs_plan_moe_scores(self.handle, body, MOE_SCORES[m.scores], int(m.identity)))
+        if m.weight_scale != 1.0:
+            self._made(L.library().gibbs_plan_moe_weight_scale(self.handle, body, m.weight_scale))
         if m.weigh == "input":
             self._made(L.library().gibbs_plan_moe_weigh_input(self.handle, body))
         return body
@@ -552,6 +620,10 @@ class NativePlan:
     def add_normed(self, norm: int, value: int) -> None:
         """x += norm(a body's delta): normed and added in one pass (float32), the delta is used up."""
         self._made(L.library().gibbs_plan_op_add_normed(self.handle, norm, value))
+
+    def weighted_sum(self, value: int, scale: float, value2: int, scale2: float) -> int:
+        """-> value: scale * delta + scale2 * delta2 of two bodies' deltas, which are used up (float32, taken where it is added)."""
+        return self._made(L.library().gibbs_plan_op_sum(self.handle, value, float(scale), value2, float(scale2)))
 
     def reinject(self) -> None:
         """x += the embedding's output (the rows as the step's first operation saw them)."""

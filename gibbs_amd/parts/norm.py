@@ -4,7 +4,7 @@ LayerNorm (`"layer"`): out = (x - mean) / sqrt(mean((x - mean)^2) + eps) * gain 
 norms a weighted sum of several residual streams (what a hyper-connected sublayer reads).
 
 RMSNorm: out = x * 1/sqrt(mean(x^2) + eps) * gain, eps inside the root, the gain multiplied
-last, no (1 + gain) offset (src/model/simd.rs:75-110,
+last, no (1 + gain) offset unless the spec names one (src/model/simd.rs:75-110,
 arch/lib/transformer.json5:9-11)."""
 from __future__ import annotations
 
@@ -19,12 +19,14 @@ from .base import Norm, Runtime, register_norm
 @register_norm("rms")
 class RMSNorm(Norm):
     def tensor_decls(self) -> List[TensorDecl]:
-        names = [self.spec.weight] + ([self.spec.scale] if self.spec.scale is not None else [])
-        return [TensorDecl(n, (self.width,), FLOAT32, init="gain") for n in names]
+        decls = [TensorDecl(self.spec.weight, (self.width,), FLOAT32, init="bias" if self.spec.offset else "gain")]
+        return decls + ([TensorDecl(self.spec.scale, (self.width,), FLOAT32, init="gain")] if self.spec.scale is not None else [])
 
     def bind(self, weights: WeightStore, rt: Runtime) -> None:
         self.rt = rt
         self.gain = weights[self.spec.weight]
+        if self.spec.offset:                 # (a weight that is stored around zero)
+            self.gain = (self.gain + self.spec.offset).contiguous()
         if self.spec.scale is not None:      # (a scale per channel on the normed row: one more factor of the gain)
             self.gain = (self.gain * weights[self.spec.scale]).contiguous()
 
