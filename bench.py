@@ -385,10 +385,38 @@ def gumozen_shape(width: int, ff: int, layers: int, vocab: int) -> dict:
     return {"architecture": "Gumozen", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": made}
 
 
+def lubavik_shape(width: int, ff: int, layers: int, vocab: int) -> dict:
+    """A Lubavik model of `layers` layers (matrix memory, attention, a pair of chunked attention and gated linear attention in turn) whose
+    sizes resemble a real model's at this width: memory heads of 128 x 128; attention heads of 64 in groups of four, whole heads
+    turned, every attention layer behind the first reading the first one's keys and values; in a pair, chunked heads of 64 over
+    values of 128 (half as many, in groups of four, chunks of 1,024) beside linear heads of 64 x 128; 64 entries of the second token table
+    a layer; a squared-relu feed-forward of the dense width in the memory layers, elsewhere 16 experts of an
+    eighth of the dense width, of which a token takes 4, beside a shared one of half the dense width."""
+    heads = max(1, width // 64)
+    half = max(1, width // 128)
+    rot = {"base": 500000.0, "dims": 64}
+    experts = {"kind": "moe", "expert": {"ff": ff // 8}, "router": {"experts": 16, "top": 4, "scale": 2.0}, "shared": {"ff": ff // 2}}
+    attention = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 64, "vdim": 64, "scale": 0.125, "rot": rot}
+    kinds = [
+        {"type": "mlstm", "mixer": {"heads": half, "dim": 128, "vdim": 128, "gate_cap": 15.0}, "mlp": {"kind": "dense", "ff": ff}},
+        {"type": "attention", "mixer": attention, "mlp": experts},
+        {"type": "parallel", "mlp": experts,
+         "mixer": {"left": {"heads": half, "kv_heads": max(1, half // 4), "dim": 64, "vdim": 128, "scale": 0.125, "mask": {"size": 1024}, "rot": rot},
+                   "right": {"heads": half, "dim": 64, "vdim": 128, "tau": 8.0}, "left_scale": 0.9, "right_scale": 0.7}},
+    ]
+    made = []
+    for i in range(layers):
+        layer = dict(kinds[i % 3])
+        if i % 3 == 1 and i > 1:
+            layer["mixer"] = dict(attention, kv_from=1)
+        made.append(layer)
+    return {"architecture": "Lubavik", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "token_side": {"dim": 64}, "layers": made}
+
+
 # design -> (its name, its shape, the closest model the framework had, that model's shape at equal sizes)
 BESIDE = {"zokepel": ("Zokepel", zokepel_shape, "LFM2", lfm2_shape), "rukosun": ("Rukosun", rukosun_shape, "LFM2", lfm2_attention_shape),
           "ruzinex": ("Ruzinex", ruzinex_shape, "LFM2", lfm2_attention_shape), "litizen": ("Litizen", litizen_shape, "Ruzinex", ruzinex_shape),
-          "gumozen": ("Gumozen", gumozen_shape, "Litizen", litizen_shape)}
+          "gumozen": ("Gumozen", gumozen_shape, "Litizen", litizen_shape), "lubavik": ("Lubavik", lubavik_shape, "Gumozen", gumozen_shape)}
 
 
 def engine_of(shape: dict, dtype: str, max_requests: int, context: int):
@@ -470,7 +498,7 @@ def main() -> int:
     ap = argparse.ArgumentParser()
     ap.add_argument("--design", choices=["lfm2"] + sorted(BESIDE), default="lfm2",
                     help="zokepel, rukosun, ruzinex: that design beside LFM2 at equal sizes instead of the headline workload; "
-                         "litizen: beside Ruzinex, gumozen: beside Litizen, the closest designs the framework had")
+                         "litizen: beside Ruzinex, gumozen: beside Litizen, lubavik: beside Gumozen, the closest designs the framework had")
     ap.add_argument("--sizes", choices=["small", "medium", "all"], default="medium", help="sizes of --design (any but lfm2)")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=128)

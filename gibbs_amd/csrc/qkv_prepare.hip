@@ -244,6 +244,102 @@ __global__ __launch_bounds__(256) void qkv_prepare_bf16x8_kernel(bf16* __restric
   put(j0, y0);
   put(j0 + half, y1);
 }
+// Eight neighbouring channels of a head, starting at channel c: the rotation of those below `rot` in interleaved pairs (rot in steps
+// of 8: all eight or none).
+__device__ __forceinline__ void turn_interleaved8(const QkvPrepareArgs& a, int p, int c, float* f) {
+  if (c >= a.rot) return;
+  const int j0 = c / 2;
+  float cs[8];
+  if (a.cs_table && p < a.table_len) {
+    const float4* t = (const float4*)(a.cs_table + (size_t)p * (a.rot / 2) + j0);
+    const float4 u = t[0], v = t[1];
+    cs[0] = u.x; cs[1] = u.y; cs[2] = u.z; cs[3] = u.w; cs[4] = v.x; cs[5] = v.y; cs[6] = v.z; cs[7] = v.w;
+  } else {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) rope_cos_sin((float)p * a.inv_freq[j0 + i], &cs[2 * i], &cs[2 * i + 1]);
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const float x = f[2 * i], y = f[2 * i + 1];
+    f[2 * i] = x * cs[2 * i] - y * cs[2 * i + 1];
+    f[2 * i + 1] = y * cs[2 * i] + x * cs[2 * i + 1];
+  }
+}
+// The cosines and sines of eight neighbouring pairs from j on: (cos, sin) in turn.
+__device__ __forceinline__ void cos_sin8(const QkvPrepareArgs& a, int p, int j, float* cs) {
+  if (a.cs_table && p < a.table_len) {
+    const float4* t = (const float4*)(a.cs_table + (size_t)p * (a.rot / 2) + j);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) { const float4 u = t[i]; cs[4 * i] = u.x; cs[4 * i + 1] = u.y; cs[4 * i + 2] = u.z; cs[4 * i + 3] = u.w; }
+  } else {
+#pragma unroll
+    for (int i = 0; i < 8; ++i) rope_cos_sin((float)p * a.inv_freq[j + i], &cs[2 * i], &cs[2 * i + 1]);
+  }
+}
+__device__ __forceinline__ void floats8(const float* p, float* f) {
+  const float4 x = *(const float4*)p, y = *(const float4*)(p + 4);
+  f[0] = x.x; f[1] = x.y; f[2] = x.z; f[3] = x.w; f[4] = y.x; f[5] = y.y; f[6] = y.z; f[7] = y.w;
+}
+// What qkv_prepare_kernel does for bfloat16 rows whose sizes come in steps of 8, heads and values of up to 128, with biases, per-head
+// norms and the rotation (no value mixing): 16 lanes share a head and hold 8 channels each, so that a value is loaded once, with its 7
+// neighbours.  In half-split pairs a channel's partner waits in another lane of the head.
+__global__ __launch_bounds__(256) void qkv_prepare_heads8_kernel(bf16* __restrict__ rows, bf16* __restrict__ kpages, bf16* __restrict__ vpages, QkvPrepareArgs a) {
+  constexpr int LPH = 16;
+  const int n = blockIdx.x, hs = blockIdx.y * (blockDim.x / LPH) + threadIdx.x / LPH, lane = threadIdx.x % LPH, c = lane * 8;
+  if (hs >= a.nh + 2 * a.nkv) return;      // (all lanes of a head leave together)
+  const bool is_q = hs < a.nh, is_k = !is_q && hs < a.nh + a.nkv;
+  const int g = is_q ? hs : (is_k ? hs - a.nh : hs - a.nh - a.nkv), size = (is_q || is_k) ? a.hd : a.vd;
+  const long off = is_q ? (long)g * a.hd : (is_k ? (long)(a.nh + g) * a.hd : (long)(a.nh + a.nkv) * a.hd + (long)g * a.vd);
+  bf16* src = rows + (size_t)n * a.ld + off;
+  const bool live = c < size;
+  const int p = a.pos[n];
+  float f[8] = {};
+  if (live) {
+    unpack_bf16x8(*(const uint4*)(src + c), f);
+    if (a.bias) {
+      float b[8];
+      floats8(a.bias + off + c, b);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) f[i] += b[i];
+    }
+  }
+  bf16* page_dst = nullptr;
+  if (!is_q && kpages) {
+    const int page = a.table[(size_t)a.row_req[n] * a.max_pages + p / a.page_size];
+    if (page >= 0 && page < a.num_pages)
+      page_dst = (is_k ? kpages : vpages) + (((size_t)page * a.nkv + g) * a.page_size + p % a.page_size) * size;
+  }
+  const float* gain = is_q ? a.q_gain : (is_k ? a.k_gain : nullptr);
+  if (gain) {
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) if (c + i < a.norm_dim) ss = fmaf(f[i], f[i], ss);
+    const float inv = 1.0f / sqrtf(group_sum<LPH>(ss) / (float)a.norm_dim + a.qk_eps);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) f[i] = c + i < a.norm_dim ? f[i] * inv * gain[c + i] : 0.f;
+  }
+  if (is_q || is_k) {
+    if (a.variant == ROPE_INTERLEAVED) {
+      turn_interleaved8(a, p, c, f);
+    } else if (a.rot) {
+      const int half = a.rot / 2;
+      const bool first = c < half, turned = c < a.rot;
+      const int from = turned ? (first ? lane + half / 8 : lane - half / 8) : lane;
+      float y[8], cs[16];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) y[i] = __shfl(f[i], from, LPH);
+      if (turned) {
+        cos_sin8(a, p, first ? c : c - half, cs);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) f[i] = first ? f[i] * cs[2 * i] - y[i] * cs[2 * i + 1] : f[i] * cs[2 * i] + y[i] * cs[2 * i + 1];
+      }
+    }
+  }
+  if (!live) return;
+  const uint4 r = pack_bf16x8(f);
+  *(uint4*)(src + c) = r;
+  if (page_dst) *(uint4*)(page_dst + c) = r;
+}
 // The heads' outputs att [N, nh * vd] (row stride ldo), in place: each head turned back by its row's position over its
 // first v_rot channels (pair m by -pos * v_inv_freq[m]; null: not turned), then multiplied element by element with
 // sigmoid(gate[n, h * gate_head + c]) (gate rows of stride ld_gate in the same type, c < vt; null: no gate).  float32 arithmetic.
@@ -295,23 +391,12 @@ __global__ __launch_bounds__(256) void qkv_prepare_whole_kernel(T* __restrict__ 
     else if constexpr (V == 8) { *(float4*)p = make_float4(f[0], f[1], f[2], f[3]); *(float4*)(p + 4) = make_float4(f[4], f[5], f[6], f[7]); }
     else *p = from_float<T>(f[0]);
   };
-  float ssq = 0.f, ssk = 0.f;
-  for (int e = threadIdx.x * V; e < nq + nk; e += blockDim.x * V) {
-    float f[V];
-    load(row + e, f);
-    float ss = 0.f;
-#pragma unroll
-    for (int i = 0; i < V; ++i) {
-      buf[e + i] = f[i];
-      ss = fmaf(f[i], f[i], ss);
-    }
-    if (e < nq) ssq += ss; else ssk += ss;
-  }
-  ssq = block_sum(ssq, scratch_q);
-  ssk = block_sum(ssk, scratch_k);               // (the barriers inside publish buf as well)
-  // (heads stored wider than they are have zeros behind: the mean counts the true channels)
-  const float inv_q = 1.0f / sqrtf(ssq / (float)(a.nh * a.norm_dim) + a.qk_eps);
-  const float inv_k = nk ? 1.0f / sqrtf(ssk / (float)(a.nkv * a.norm_dim) + a.qk_eps) : 0.f;
+  auto floats = [&](const float* p, float* f) {       // V neighbouring float32 values
+    if constexpr (V == 8) {
+      const float4 x = *(const float4*)p, y = *(const float4*)(p + 4);
+      f[0] = x.x; f[1] = x.y; f[2] = x.z; f[3] = x.w; f[4] = y.x; f[5] = y.y; f[6] = y.z; f[7] = y.w;
+    } else f[0] = *p;
+  };
   const int p = a.pos[n];
   int page = -1, at = 0;
   if (nk && kpages) {
@@ -319,41 +404,174 @@ __global__ __launch_bounds__(256) void qkv_prepare_whole_kernel(T* __restrict__ 
     at = p % a.page_size;
     if (page >= a.num_pages) page = -1;          // (the host never asks for another; never write outside the pool)
   }
+  float ssq = 0.f, ssk = 0.f;
+  for (int e = threadIdx.x * V; e < nq + nk; e += blockDim.x * V) {
+    float f[V];
+    load(row + e, f);
+    float ss = 0.f;
+    if constexpr (V == 8) {
+      *(float4*)(buf + e) = make_float4(f[0], f[1], f[2], f[3]);
+      *(float4*)(buf + e + 4) = make_float4(f[4], f[5], f[6], f[7]);
+    } else buf[e] = f[0];
+#pragma unroll
+    for (int i = 0; i < V; ++i) ss = fmaf(f[i], f[i], ss);
+    if (e < nq) ssq += ss; else ssk += ss;
+  }
+  if (page >= 0)
+    for (int e = threadIdx.x * V; e < a.nkv * a.vd; e += blockDim.x * V) {
+      float f[V];
+      load(row + nq + nk + e, f);
+      store(vpages + (((size_t)page * a.nkv + e / a.vd) * a.page_size + at) * a.vd + e % a.vd, f);
+    }
+  ssq = block_sum(ssq, scratch_q);
+  ssk = block_sum(ssk, scratch_k);               // (the barriers inside publish buf as well)
+  // (heads stored wider than they are have zeros behind: the mean counts the true channels)
+  const float inv_q = 1.0f / sqrtf(ssq / (float)(a.nh * a.norm_dim) + a.qk_eps);
+  const float inv_k = nk ? 1.0f / sqrtf(ssk / (float)(a.nkv * a.norm_dim) + a.qk_eps) : 0.f;
+  const bool half_split = a.variant == ROPE_HALF_SPLIT, from_table = a.cs_table && p < a.table_len;
   for (int e = threadIdx.x * V; e < nq + nk; e += blockDim.x * V) {
     const bool is_q = e < nq;
     const int rel = is_q ? e : e - nq, head = rel / a.hd, c = rel % a.hd;
     const float inv = is_q ? inv_q : inv_k;
-    const float* gain = is_q ? a.q_gain + rel : a.k_gain + rel;
-    float f[V];
+    const float* gain = (is_q ? a.q_gain : a.k_gain) + rel;
+    float f[V], g[V];
+    floats(buf + e, f);
+    floats(gain, g);
 #pragma unroll
-    for (int i = 0; i < V; ++i) {
-      const int ch = c + i;
-      float x = buf[e + i] * inv * gain[i];
-      if (ch < 2 * half) {
-        const int j = a.variant == ROPE_HALF_SPLIT ? (ch < half ? ch : ch - half) : ch / 2;
-        const bool first = a.variant == ROPE_HALF_SPLIT ? ch < half : (ch & 1) == 0;
-        const int step = a.variant == ROPE_HALF_SPLIT ? (first ? half : -half) : (first ? 1 : -1);
-        const float y = buf[e + i + step] * inv * gain[i + step];
+    for (int i = 0; i < V; ++i) f[i] *= inv * g[i];
+    if (V == 8 && half_split && half % 8 == 0 && c < 2 * half) {       // the partners are 8 neighbours as well
+      const bool first = c < half;
+      const int step = first ? half : -half, j = first ? c : c - half;
+      float y[V], cs[2 * V];
+      floats(buf + e + step, y);
+      floats(gain + step, g);
+      if (from_table) {
+        const float* t = (const float*)(a.cs_table + (size_t)p * half + j);
+        floats(t, cs);
+        floats(t + V, cs + V);
+      } else {
+#pragma unroll
+        for (int i = 0; i < V; ++i) rope_cos_sin((float)p * a.inv_freq[j + i], &cs[2 * i], &cs[2 * i + 1]);
+      }
+#pragma unroll
+      for (int i = 0; i < V; ++i) {
+        const float partner = y[i] * (inv * g[i]);
+        f[i] = first ? f[i] * cs[2 * i] - partner * cs[2 * i + 1] : f[i] * cs[2 * i] + partner * cs[2 * i + 1];
+      }
+    } else if (c < 2 * half) {
+#pragma unroll
+      for (int i = 0; i < V; ++i) {
+        const int ch = c + i;
+        if (ch >= 2 * half) continue;
+        const int j = half_split ? (ch < half ? ch : ch - half) : ch / 2;
+        const bool first = half_split ? ch < half : (ch & 1) == 0;
+        const int step = half_split ? (first ? half : -half) : (first ? 1 : -1);
+        const float partner = buf[e + i + step] * (inv * gain[i + step]);
         float cs, sn;
-        if (a.cs_table && p < a.table_len) {
+        if (from_table) {
           const float2 t = a.cs_table[(size_t)p * half + j];
           cs = t.x;
           sn = t.y;
         } else {
           rope_cos_sin((float)p * a.inv_freq[j], &cs, &sn);
         }
-        x = first ? x * cs - y * sn : x * cs + y * sn;
+        f[i] = first ? f[i] * cs - partner * sn : f[i] * cs + partner * sn;
       }
-      f[i] = x;
     }
     store(row + e, f);
     if (!is_q && page >= 0) store(kpages + (((size_t)page * a.nkv + head) * a.page_size + at) * a.hd + c, f);
   }
-  if (page < 0) return;
-  for (int e = threadIdx.x * V; e < a.nkv * a.vd; e += blockDim.x * V) {
-    float f[V];
-    load(row + nq + nk + e, f);
-    store(vpages + (((size_t)page * a.nkv + e / a.vd) * a.page_size + at) * a.vd + e % a.vd, f);
+}
+// The same for bfloat16 rows in steps of 8 (the rotated part in steps of 16 in half-split pairs, of 8 in interleaved ones): a thread
+// holds the channels j .. j + 7 of a head and their partners, or 8 channels that have none or hold both, in registers over the sums.
+// R: such items a thread holds.
+template <int R>
+__global__ __launch_bounds__(256) void qkv_prepare_whole8_kernel(bf16* __restrict__ rows, bf16* __restrict__ kpages, bf16* __restrict__ vpages, QkvPrepareArgs a) {
+  __shared__ float2 scratch[4];
+  const int n = blockIdx.x, tid = threadIdx.x, lane = tid % WAVE, wave = tid / WAVE;
+  const int half = a.variant == ROPE_HALF_SPLIT ? a.rot / 2 : 0, pairs = half / 8, per_head = a.hd / 8 - pairs, items = (a.nh + a.nkv) * per_head;
+  bf16* row = rows + (size_t)n * a.ld;
+  const int p = a.pos[n];
+  uint4 x[R][2];
+  int head[R], c[R];
+  float ssq = 0.f, ssk = 0.f;
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    const int it = tid + r * 256;
+    head[r] = it / per_head;
+    const int sub = it % per_head;
+    c[r] = sub < pairs ? sub * 8 : (sub + pairs) * 8;
+    if (it >= items) continue;
+    const bf16* at = row + head[r] * a.hd + c[r];
+    x[r][0] = *(const uint4*)at;
+    if (sub < pairs) x[r][1] = *(const uint4*)(at + half);
+  }
+  int page = -1, slot = 0;
+  if (a.nkv && kpages) {
+    page = a.table[(size_t)a.row_req[n] * a.max_pages + p / a.page_size];
+    slot = p % a.page_size;
+    if (page >= a.num_pages) page = -1;          // (the host never asks for another; never write outside the pool)
+  }
+  if (page >= 0)
+    for (int e = tid * 8; e < a.nkv * a.vd; e += 256 * 8)
+      *(uint4*)(vpages + (((size_t)page * a.nkv + e / a.vd) * a.page_size + slot) * a.vd + e % a.vd) = *(const uint4*)(row + (a.nh + a.nkv) * a.hd + e);
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    if (tid + r * 256 >= items) continue;
+    float f[8], ss = 0.f;
+    unpack_bf16x8(x[r][0], f);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) ss = fmaf(f[i], f[i], ss);
+    if (c[r] < half) {
+      unpack_bf16x8(x[r][1], f);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) ss = fmaf(f[i], f[i], ss);
+    }
+    if (head[r] < a.nh) ssq += ss; else ssk += ss;
+  }
+  ssq = wave_sum(ssq);
+  ssk = wave_sum(ssk);
+  if (lane == 0) scratch[wave] = make_float2(ssq, ssk);
+  __syncthreads();
+  ssq = ssk = 0.f;
+#pragma unroll
+  for (int w = 0; w < 4; ++w) { ssq += scratch[w].x; ssk += scratch[w].y; }
+  const float inv_q = 1.0f / sqrtf(ssq / (float)(a.nh * a.norm_dim) + a.qk_eps);
+  const float inv_k = a.nkv ? 1.0f / sqrtf(ssk / (float)(a.nkv * a.norm_dim) + a.qk_eps) : 0.f;
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    if (tid + r * 256 >= items) continue;
+    const bool is_q = head[r] < a.nh;
+    const int g = is_q ? head[r] : head[r] - a.nh;
+    const float inv = is_q ? inv_q : inv_k;
+    const float* gain = (is_q ? a.q_gain : a.k_gain) + g * a.hd + c[r];
+    bf16* at = row + head[r] * a.hd + c[r];
+    bf16* page_at = !is_q && page >= 0 ? kpages + (((size_t)page * a.nkv + g) * a.page_size + slot) * a.hd + c[r] : nullptr;
+    float f[8], w[8];
+    unpack_bf16x8(x[r][0], f);
+    floats8(gain, w);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) f[i] *= inv * w[i];
+    if (c[r] < half) {
+      float y[8], cs[16], u[8];
+      unpack_bf16x8(x[r][1], y);
+      floats8(gain + half, w);
+      cos_sin8(a, p, c[r], cs);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        y[i] *= inv * w[i];
+        u[i] = y[i] * cs[2 * i] + f[i] * cs[2 * i + 1];
+        f[i] = f[i] * cs[2 * i] - y[i] * cs[2 * i + 1];
+      }
+      const uint4 v = pack_bf16x8(u);
+      *(uint4*)(at + half) = v;
+      if (page_at) *(uint4*)(page_at + half) = v;
+    } else if (a.variant == ROPE_INTERLEAVED) {
+      turn_interleaved8(a, p, c[r], f);
+    }
+    const uint4 v = pack_bf16x8(f);
+    *(uint4*)at = v;
+    if (page_at) *(uint4*)page_at = v;
   }
 }
 }  // namespace
@@ -392,6 +610,12 @@ GIBBS_EXPORT int gibbs_qkv_prepare_full(void* rows, long ld, void* kpages, void*
   const bool narrow = hd <= 128 && vd <= 128;      // four heads a wave
   const int per_block = narrow ? 16 : 4;
   const dim3 grid(n_rows, ceil_div(nh + 2 * nkv, per_block));
+  const bool pairs8 = !inv_freq || (rot % (variant == ROPE_HALF_SPLIT ? 16 : 8) == 0 && ((uintptr_t)cs_table % 16) == 0);
+  if (dtype == GIBBS_BF16 && narrow && keep_mode == KEEP_NONE && !v_from_k && !v_inv_freq && hd % 8 == 0 && vd % 8 == 0 && ld % 8 == 0 && pairs8 &&
+      ((uintptr_t)rows % 16) == 0 && ((uintptr_t)bias % 16) == 0 && (!kpages || (((uintptr_t)kpages % 16) == 0 && ((uintptr_t)vpages % 16) == 0))) {
+    qkv_prepare_heads8_kernel<<<grid, 256, 0, stream>>>((bf16*)rows, (bf16*)kpages, (bf16*)vpages, a);
+    GIBBS_LAUNCH_STATUS("qkv_prepare");
+  }
   if (dtype == GIBBS_F32) {
     if (narrow) qkv_prepare_kernel<float, 16><<<grid, 256, 0, stream>>>((float*)rows, (float*)kpages, (float*)vpages, (float*)keep, a);
     else qkv_prepare_kernel<float, 64><<<grid, 256, 0, stream>>>((float*)rows, (float*)kpages, (float*)vpages, (float*)keep, a);
@@ -430,7 +654,21 @@ GIBBS_EXPORT int gibbs_qkv_prepare_whole(void* rows, long ld, void* kpages, void
   a.inv_freq = inv_freq; a.rot = inv_freq ? rot : 0; a.variant = variant; a.cs_table = (const float2*)cs_table; a.table_len = cs_table && inv_freq ? table_len : 0;
   a.pos = pos; a.row_req = row_req; a.table = table; a.max_pages = max_pages; a.page_size = page_size; a.num_pages = num_pages;
   a.nh = nh; a.nkv = nkv; a.hd = hd; a.vd = vd; a.ld = ld; a.q_gain = q_gain; a.k_gain = k_gain; a.qk_eps = eps; a.norm_dim = norm_dim;
-  const bool x8 = hd % 8 == 0 && vd % 8 == 0 && ld % 8 == 0 && ((uintptr_t)rows % 16) == 0 && (!kpages || (((uintptr_t)kpages % 16) == 0 && ((uintptr_t)vpages % 16) == 0));
+  const bool x8 = hd % 8 == 0 && vd % 8 == 0 && ld % 8 == 0 && ((uintptr_t)rows % 16) == 0 && ((uintptr_t)q_gain % 16) == 0 && ((uintptr_t)k_gain % 16) == 0 &&
+                  ((uintptr_t)cs_table % 16) == 0 && (!kpages || (((uintptr_t)kpages % 16) == 0 && ((uintptr_t)vpages % 16) == 0));
+  const bool pairs8 = !inv_freq || rot % (variant == ROPE_HALF_SPLIT ? 16 : 8) == 0;
+  if (dtype == GIBBS_BF16 && x8 && pairs8) {      // (a head's items: its pairs of eight channels and what is not in pairs)
+    const long items = (long)(nh + nkv) * (hd / 8 - (a.rot && variant == ROPE_HALF_SPLIT ? rot / 16 : 0));
+#define WHOLE8(R)                                                                                                        \
+  do {                                                                                                                   \
+    qkv_prepare_whole8_kernel<R><<<n_rows, 256, 0, stream>>>((bf16*)rows, (bf16*)kpages, (bf16*)vpages, a);              \
+    GIBBS_LAUNCH_STATUS("qkv_prepare_whole");                                                                            \
+  } while (0)
+    if (items <= 256) WHOLE8(1);
+    if (items <= 512) WHOLE8(2);
+    if (items <= 1024) WHOLE8(4);
+#undef WHOLE8
+  }
 #define PREPARE_WHOLE(T, V)                                                                                                              \
   do {                                                                                                                                   \
     static bool raised = false;                                                                                                          \

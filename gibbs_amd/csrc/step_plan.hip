@@ -1284,7 +1284,10 @@ struct MatrixLstmBody : Body {
     if (lead > 0) walk(nullptr, a.slot, lead);
     if (rest > 0 && a.max_q >= WALKED_ROWS && gibbs_matrix_lstm_chunks_take(D, V)) {
       const Matrix rows{(char*)h + (long)lead * W * e.esize, nullptr, rest, W};
-      float* gates = (float*)e.linear(w_gates, rows, 2 * H, true, false, false, nullptr);
+      float* gates = (float*)e.take((long)2 * H * rest * 4);
+      const int piece = 2 * H > SKINNY_ROWS_F32_OUT ? 32 : 2 * H;      // (what the few-row product takes)
+      for (int o = 0; o < 2 * H; o += piece)
+        e.linear_into((const char*)w_gates + (long)o * W * e.esize, rows, std::min(piece, 2 * H - o), true, false, gates + (long)o * rest);
       float* work = (float*)e.take(gibbs_matrix_lstm_chunks_workspace(rest, reqs, H, D, V) * 4);
       RUN(e, gibbs_matrix_lstm_chunks(raw, in.O, off_q, off_k, off_v, off_g, h, W, w_gates, b_gates, gain, cap, eps, q_scale, rule_state, norm_state, slot_stride,
                                       a.cu + lead, a.slot + lead, y, gates, work, e.p.dtype, rest, reqs, H, D, V, a.stream));
