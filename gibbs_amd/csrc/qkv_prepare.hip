@@ -315,8 +315,14 @@ __global__ __launch_bounds__(256) void qkv_prepare_heads8_kernel(bf16* __restric
 #pragma unroll
     for (int i = 0; i < 8; ++i) if (c + i < a.norm_dim) ss = fmaf(f[i], f[i], ss);
     const float inv = 1.0f / sqrtf(group_sum<LPH>(ss) / (float)a.norm_dim + a.qk_eps);
+    float w[8] = {};
+    if (c + 8 <= a.norm_dim) floats8(gain + c, w);
+    else {
 #pragma unroll
-    for (int i = 0; i < 8; ++i) f[i] = c + i < a.norm_dim ? f[i] * inv * gain[c + i] : 0.f;
+      for (int i = 0; i < 8; ++i) if (c + i < a.norm_dim) w[i] = gain[c + i];
+    }
+#pragma unroll
+    for (int i = 0; i < 8; ++i) f[i] = f[i] * inv * w[i];
   }
   if (is_q || is_k) {
     if (a.variant == ROPE_INTERLEAVED) {
@@ -612,7 +618,8 @@ GIBBS_EXPORT int gibbs_qkv_prepare_full(void* rows, long ld, void* kpages, void*
   const dim3 grid(n_rows, ceil_div(nh + 2 * nkv, per_block));
   const bool pairs8 = !inv_freq || (rot % (variant == ROPE_HALF_SPLIT ? 16 : 8) == 0 && ((uintptr_t)cs_table % 16) == 0);
   if (dtype == GIBBS_BF16 && narrow && keep_mode == KEEP_NONE && !v_from_k && !v_inv_freq && hd % 8 == 0 && vd % 8 == 0 && ld % 8 == 0 && pairs8 &&
-      ((uintptr_t)rows % 16) == 0 && ((uintptr_t)bias % 16) == 0 && (!kpages || (((uintptr_t)kpages % 16) == 0 && ((uintptr_t)vpages % 16) == 0))) {
+      ((uintptr_t)rows % 16) == 0 && ((uintptr_t)bias % 16) == 0 && ((uintptr_t)q_gain % 16) == 0 && ((uintptr_t)k_gain % 16) == 0 &&
+      (!kpages || (((uintptr_t)kpages % 16) == 0 && ((uintptr_t)vpages % 16) == 0))) {
     qkv_prepare_heads8_kernel<<<grid, 256, 0, stream>>>((bf16*)rows, (bf16*)kpages, (bf16*)vpages, a);
     GIBBS_LAUNCH_STATUS("qkv_prepare");
   }
