@@ -261,10 +261,66 @@ def _pad8(n):
     return -(-n // 8) * 8
 
 
+def _cos_sin(freq, length):
+    """The table of cosines and sines of the first `length` positions; positions behind it have theirs computed."""
+    angle = (np.arange(length, dtype=np.float32)[:, None] * freq[None, :]).astype(np.float32).astype(np.float64)
+    return np.stack([np.cos(angle), np.sin(angle)], axis=-1).astype(np.float32)
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("variant", [0, 1])
+@pytest.mark.parametrize("sizes", [(6, 3, 10, 14, 6, 10, 14), (4, 2, 24, 40, 16, 48, 48), (5, 1, 40, 128, 32, 128, 128), (8, 2, 64, 64, 64, 64, 64), (7, 7, 20, 12, 8, 32, 32)])
+def test_rows_with_biases_and_normed_heads(sizes, variant, dtype):
+    """Biases, q and k heads divided by their own root mean square, a gain that the heads share, the rotation of part of a head in both
+    layouts, keys and values in their pages; heads stored wider than they are."""
+    from gibbs_amd.ops.lib import call, dtype_code, ptr, stream
+    rng = np.random.default_rng(5)
+    H, G, D, V, rot, ks, vs = sizes
+    ps, places = 16, [0, 15, 16, 250, 3000]
+    n = len(places)
+    ld = (H + G) * ks + G * vs + 8
+    spans = [(0, H, ks, D), (H * ks, G, ks, D), ((H + G) * ks, G, vs, V)]
+    r, bias = np.zeros((n, ld)), np.zeros((H + G) * ks + G * vs)
+    for at, heads, stored, true in spans:
+        for h in range(heads):
+            r[:, at + h * stored:at + h * stored + true] = rng.normal(size=(n, true)) * (0.3 + h)
+            bias[at + h * stored:at + h * stored + true] = rng.normal(size=true)
+    rows = _dev(r, dtype)
+    r64, b64 = _f64(rows), bias.astype(np.float32).astype(np.float64)
+    gains = [(rng.normal(size=D) + 1.0).astype(np.float32) for _ in range(2)]
+    base = 500.0
+    freq = np.array([base ** (-2.0 * i / rot) for i in range(rot // 2)]).astype(np.float32)
+    n_pages = 3000 // ps + 1
+    kpages = torch.full((n_pages, G, ps, ks), 7.0, dtype=dtype, device="cuda")
+    vpages = torch.full((n_pages, G, ps, vs), 7.0, dtype=dtype, device="cuda")
+    table = torch.arange(n_pages - 1, -1, -1, dtype=torch.int32, device="cuda").view(1, n_pages).contiguous()
+    turns, dev_gains = _dev(_cos_sin(freq, 100)), [_dev(np.pad(g, (0, ks - D))) for g in gains]
+    call("gibbs_qkv_prepare_full", ptr(rows), ld, ptr(kpages), ptr(vpages), dtype_code(dtype), ptr(_dev(bias)), ptr(_dev(freq)), rot, variant, ptr(turns), 100,
+         None, 0, V, None, ptr(_dev(places, torch.int32)), ptr(_dev([0] * n, torch.int32)), ptr(table), n_pages, ps, n_pages, n, H, G, ks, vs,
+         ptr(dev_gains[0]), ptr(dev_gains[1]), 1e-5, D, 0, None, 0, stream())
+    got = _f64(rows)
+    tol = 1e-4 if dtype == torch.float32 else 0.1
+    want = []
+    for which, (at, heads, stored, true) in enumerate(spans):
+        x = (r64[:, at:at + heads * stored] + b64[at:at + heads * stored]).reshape(n, heads, stored)[:, :, :true]
+        if which < 2:
+            x = Z.rotate(Z.rms_unit(x, 1e-5) * gains[which].astype(np.float64), places, base, rot, neighbours=variant == 1)
+        want.append(x)
+        have = got[:, at:at + heads * stored].reshape(n, heads, stored)
+        assert (np.abs(have[:, :, :true] - x) <= tol * np.maximum(1.0, np.abs(x) / 4)).all()
+        assert not have[:, :, true:].any()
+    assert np.array_equal(got[:, (H + G) * ks + G * vs:], r64[:, (H + G) * ks + G * vs:])
+    for pages, x, true in ((kpages, want[1], D), (vpages, want[2], V)):
+        for row, p in enumerate(places):
+            have = _f64(pages[n_pages - 1 - p // ps, :, p % ps])
+            assert (np.abs(have[:, :true] - x[row]) <= tol * np.maximum(1.0, np.abs(x[row]) / 4)).all() and not have[:, true:].any()
+        assert int((pages == 7.0).all(-1).sum()) == (n_pages * ps - n) * G
+
+
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("variant", [0, 1])
 @pytest.mark.parametrize("sizes", [(6, 3, 10, 14, 6, 10, 14), (4, 2, 24, 40, 24, 48, 48), (8, 2, 64, 128, 32, 128, 128), (3, 0, 16, 16, 16, 16, 16), (2, 1, 5, 3, 0, 5, 3),
-                                   (40, 8, 64, 64, 64, 64, 64)])
+                                   (40, 8, 64, 64, 64, 64, 64), (72, 16, 64, 32, 48, 64, 64), (160, 8, 64, 64, 64, 64, 64)])
 def test_rows_normed_over_the_whole_projection(sizes, variant, dtype):
     """q and k divided by the root mean square of all their heads at once, a gain per channel, the rotation of both layouts, keys and
     values in their pages on both sides of page borders and far out; heads stored wider than they are; queries alone (no kv heads)."""
@@ -293,9 +349,10 @@ def test_rows_normed_over_the_whole_projection(sizes, variant, dtype):
     kpages = torch.full((n_pages, max(G, 1), ps, ks), 7.0, dtype=dtype, device="cuda")
     vpages = torch.full((n_pages, max(G, 1), ps, vs), 7.0, dtype=dtype, device="cuda")
     table = torch.arange(n_pages - 1, -1, -1, dtype=torch.int32, device="cuda").view(1, n_pages).contiguous()
+    turns = _dev(_cos_sin(freq, 100)) if rot else None
     call("gibbs_qkv_prepare_whole", ptr(rows), ld, ptr(kpages) if G else None, ptr(vpages) if G else None, dtype_code(dtype), ptr(_dev(gains[0])), ptr(_dev(gains[1])) if G else None,
-         1e-5, D, ptr(_dev(freq)) if rot else None, rot, variant, None, 0, ptr(_dev(places, torch.int32)), ptr(_dev([0] * n, torch.int32)), ptr(table), n_pages, ps, n_pages,
-         n, H, G, ks, vs, stream())
+         1e-5, D, ptr(_dev(freq)) if rot else None, rot, variant, ptr(turns) if rot else None, 100,
+         ptr(_dev(places, torch.int32)), ptr(_dev([0] * n, torch.int32)), ptr(table), n_pages, ps, n_pages, n, H, G, ks, vs, stream())
 
     def want_of(at, heads, g):
         x = r64[:, at:at + heads * ks].reshape(n, heads, ks)[:, :, :D]
